@@ -22,7 +22,9 @@ LIB = os.path.join(PKG, "libsli.so")
 ROCM = os.environ.get("ROCM_PATH", "/opt/rocm")
 ARCH = os.environ.get("SLI_OFFLOAD_ARCH", "gfx950")
 
-CXXFLAGS = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-Wall", "-Wno-unused-function",
+# no packed fp32 instructions (v_pk_add/mul/fma_f32): some of their forms gave wrong results on these GPUs now and then
+DEVFLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+CXXFLAGS = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", *DEVFLAGS, "-Wall", "-Wno-unused-function",
             "-I", os.path.join(ROOT, "include"), "-I", os.path.join(ROOT, "include", "base"),
             "-I", os.path.join(ROOT, "include", "memory"), "-I", os.path.join(ROOT, "include", "op"),
             "-I", os.path.join(ROOT, "include", "model"), "-I", os.path.join(ROOT, "include", "kernel")]
@@ -74,14 +76,28 @@ def build(force: bool = False, jobs: int | None = None, verbose: bool = False, v
         objs = list(ex.map(lambda s: _compile(s, force or variant is not None, build_dir, tuple(defines)), srcs))
     newest = max(os.path.getmtime(o) for o in objs)
     if force or variant is not None or not os.path.exists(lib) or os.path.getmtime(lib) < newest:
-        cmd = ["hipcc", f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", lib, *objs,
+        part = f"{lib}.tmp{os.getpid()}"  # renamed when whole: no process loads half a library
+        cmd = ["hipcc", f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", part, *objs,
                "-L", os.path.join(ROCM, "lib"), "-lrccl", f"-Wl,-rpath,{os.path.join(ROCM, 'lib')}"]
         r = subprocess.run(cmd, capture_output=True, text=True)
         if r.returncode != 0:
             raise RuntimeError(f"link failed: {' '.join(cmd)}\n{r.stdout}\n{r.stderr}")
+        os.replace(part, lib)
     if verbose:
         print(f"built {lib}")
     return lib
+
+
+def ensure() -> str:
+    """Build libsli.so where it is missing (a fresh checkout); one process at a time, the others wait for it."""
+    if not os.path.exists(LIB):
+        import fcntl
+        os.makedirs(BUILD, exist_ok=True)
+        with open(os.path.join(BUILD, "lock"), "w") as f:
+            fcntl.flock(f, fcntl.LOCK_EX)
+            if not os.path.exists(LIB):
+                build()
+    return LIB
 
 
 def main(argv=None) -> int:
