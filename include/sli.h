@@ -286,6 +286,52 @@ int sli_tp_group_prefill(sli_tp_group* g, const int32_t* ids, int32_t n);
 int sli_tp_group_predict_prefill(sli_tp_group* g, const int32_t* prompt, int32_t n_prompt, int32_t max_length,
                                  int32_t* tokens_out, float* logits_out);
 
+/* ---------------------------------------------------------------- block-stack models
+ * A decoder described by data, behind the same sli_model handle and decode loop as the Llama models: n_blocks
+ * parallel blocks x += residual_mult * (mixer(c1) + ff(c2)), c1 / c2 = the RMS-normed rows (one gain per sublayer)
+ * after a causal per-channel convolution of `taps` taps that is added to its input; blocks loop_start ..
+ * loop_stop - 1 run loop_times times in a row (same weights, one cache or state per run).
+ * Mixers: SLI_MIX_ATTENTION, causal grouped-query softmax attention without rotation, scores (q . k) * scale
+ * - r1 ln(1 + r2 distance) and a sink per head; SLI_MIX_RETENTION, linear attention with a fixed decay per head
+ * (decay: the retention blocks' values, concatenated in block order), rotate-half positions on the first rot_dims
+ * dims, the output normalised per head and gated by silu. Feed-forward (ff > 0): g = min(gate, ff_limit),
+ * u = clamp(up, +-ff_limit), down(g sigmoid(1.702 g) (u + 1)).
+ * Weights: SLI_DT_F16 (bfloat16 checkpoints: every bfloat16 value of magnitude 2^-14 .. 65504 is kept exactly) with
+ * an fp16 cache, or SLI_DT_F32 with an fp32 cache (true fp32 throughout). Norms, convolutions, scores, softmax,
+ * recurrent state and residual are fp32 in both. */
+typedef enum { SLI_MIX_ATTENTION = 0, SLI_MIX_RETENTION = 1 } sli_mixer_kind;
+typedef struct {
+    int32_t mixer; /* sli_mixer_kind */
+    int32_t heads, kv_heads, dim, vdim;
+    float scale;      /* attention */
+    int32_t rot_dims; /* retention */
+    double rot_base;
+    int32_t ff;       /* 0: no feed-forward */
+    float ff_limit;
+} sli_block_desc;
+typedef struct {
+    int32_t vocab, width, n_blocks, loop_start, loop_stop, loop_times, taps;
+    float eps, emb_scale, residual_mult;
+    const sli_block_desc* blocks;
+    const float* decay;
+    int32_t w_dtype; /* SLI_DT_F16 or SLI_DT_F32 */
+    int32_t max_len, batch, device;
+} sli_stack_config;
+int sli_stack_create(const sli_stack_config* cfg, sli_model** out);
+/* One tensor as full fp32 [n]: embed, head, final.norm, l<i>.{norm1,norm2,canon1,canon2}, l<i>.mix.{q,k,v,o} and
+ * {r1,r2,sink} (attention) or {g} (retention), l<i>.mlp.{gate,up,down}; matrices [out][in]. */
+int sli_stack_set_tensor(sli_model* m, const char* name, const float* host, int64_t n);
+/* Feed the next tokens of n sequences as one batch: sequence slot slots[i] gets lens[i] tokens (concatenated in
+ * `tokens`) from position starts[i] on (0: a new sequence, whatever the slot held; else the position its earlier
+ * tokens ended at). want_n[i] places among entry i's tokens (concatenated in `want`, ascending) get logits, written to
+ * logits [sum want_n][vocab] in that order. hidden (nullable, for inspection): the residual rows after every block
+ * run, [runs][sum lens][width]. */
+int sli_model_feed(sli_model* m, int32_t n, const int32_t* slots, const int32_t* starts, const int32_t* lens,
+                   const int32_t* tokens, const int32_t* want_n, const int32_t* want, float* logits, float* hidden);
+int sli_stack_runs(const sli_model* m); /* block runs of one forward pass (loops counted) */
+/* sli_model_prefill for every sequence of a block-stack model's batch at once (prompts [batch][ld]). */
+int sli_model_prefill_batch(sli_model* m, const int32_t* prompts, const int32_t* lens, int32_t ld);
+
 /* Roofline probe: replays the step's weight-streaming (GEMV) kernels `iters` times between HIP events
  * on the model's stream; returns mean device time per GEMV launch, algorithmic bytes per launch and
  * the launches per step. */

@@ -42,6 +42,18 @@ class ShardWindow(ctypes.Structure):
     _fields_ = [(n, c_i32) for n in ("row_lo", "n_rows", "col_lo", "n_cols", "full_cols", "dst_row_off")]
 
 
+class BlockDesc(ctypes.Structure):
+    _fields_ = [(n, c_i32) for n in ("mixer", "heads", "kv_heads", "dim", "vdim")] + \
+               [("scale", c_f), ("rot_dims", c_i32), ("rot_base", c_d), ("ff", c_i32), ("ff_limit", c_f)]
+
+
+class StackConfig(ctypes.Structure):
+    _fields_ = [(n, c_i32) for n in ("vocab", "width", "n_blocks", "loop_start", "loop_stop", "loop_times", "taps")] + \
+               [(n, c_f) for n in ("eps", "emb_scale", "residual_mult")] + \
+               [("blocks", ctypes.POINTER(BlockDesc)), ("decay", P_f)] + \
+               [(n, c_i32) for n in ("w_dtype", "max_len", "batch", "device")]
+
+
 # name -> (restype, argtypes)
 _SIGS = {
     "sli_version": (c_int, []),
@@ -103,6 +115,11 @@ _SIGS = {
     "sli_model_get_kv": (c_int, [c_vp, c_i32, c_i32, c_i32, c_vp]),
     "sli_model_get_kv_seq": (c_int, [c_vp, c_i32, c_i32, c_i32, c_i32, c_vp]),
     "sli_model_get_weight": (c_int, [c_vp, c_i32, c_i32, c_vp, c_i64]),
+    "sli_stack_create": (c_int, [ctypes.POINTER(StackConfig), ctypes.POINTER(c_vp)]),
+    "sli_stack_set_tensor": (c_int, [c_vp, ctypes.c_char_p, c_vp, c_i64]),
+    "sli_stack_runs": (c_int, [c_vp]),
+    "sli_model_feed": (c_int, [c_vp, c_i32, c_vp, c_vp, c_vp, c_vp, c_vp, c_vp, c_vp, c_vp]),
+    "sli_model_prefill_batch": (c_int, [c_vp, c_vp, c_vp, c_i32]),
     "sli_model_stream": (c_int, [c_vp, ctypes.POINTER(c_vp)]),
     "sli_model_step_bytes": (c_int, [c_vp, P_d, P_d]),
     "sli_model_time_gemv": (c_int, [c_vp, c_i32, P_d, P_d, P_i32]),

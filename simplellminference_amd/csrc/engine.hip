@@ -29,6 +29,7 @@
 #include "comm_wait.h"
 #include "common.h"
 #include "gemv.h"
+#include "hybrid.h"
 #include "oneshot.h"
 #include "ops_internal.h"
 #include "prefill.h"
@@ -57,6 +58,7 @@ struct LayerW {
 
 struct sli_model {
     sli_model_config c{};
+    sli::BlockStack* bs = nullptr;  // a block-stack model (hybrid.h): its forward pass; null for Llama models
     hipStream_t stream = nullptr;
     bool own_stream = true;  // false for the ranks of an in-process group (they share the group's stream)
     sli_tp_group* group = nullptr;  // in-process tensor-parallel group this rank belongs to (or null)
@@ -1223,6 +1225,7 @@ struct StepRecorder {
 
 #define SLI_DISPATCH(m, FN, ...)                                                                        \
     ([&]() -> int {                                                                                     \
+        if ((m)->bs) return fail(SLI_ERR_STATE, "not available for block-stack models");                \
         const int wd = (m)->c.w_dtype, kd = (m)->c.kv_dtype;                                            \
         if (wd == SLI_DT_F16 && kd == SLI_DT_F16) return StepRecorder<__half, __half>::FN(__VA_ARGS__); \
         if (wd == SLI_DT_F16 && kd == SLI_DT_F32) return StepRecorder<__half, float>::FN(__VA_ARGS__);  \
@@ -1276,7 +1279,30 @@ static int bg_sync_tiles(sli_model* m) {
     return SLI_OK;
 }
 
+// A block-stack model's step: its forward pass (hybrid.h), then the argmax keys and the state update every model
+// shares
+static int record_stack(sli_model* m) {
+    hipStream_t s = m->stream;
+    int nkeys = 0;
+    SLI_TRY(hy_record_step(m->bs, m->st, m->B, m->logits, m->keys, m->key_ld, &nkeys));
+    if (m->B == 1) {
+        hipLaunchKernelGGL(keyreduce_kernel<true>, dim3(1), dim3(kKeyThreads), 0, s, m->keys, nkeys, m->st, m->prompt,
+                           m->hist, m->T);
+    } else {
+        hipLaunchKernelGGL(keyreduce_batch_kernel, dim3(m->B), dim3(256), 0, s, m->keys, m->key_ld, nkeys, m->bkeys);
+        SLI_HIP(hipGetLastError());
+        hipLaunchKernelGGL(finalize_batch_kernel, dim3(1), dim3(64), 0, s, m->st, m->bkeys, m->prompt, m->hist, m->T,
+                           m->B);
+    }
+    SLI_HIP(hipGetLastError());
+    return SLI_OK;
+}
+
 static int capture(sli_model* m) {
+    if (m->bs) {
+        SLI_TRY(hy_prepare(m->bs));
+        return capture_graph(m->stream, m->graph, m->graph_exec, [&]() { return record_stack(m); });
+    }
     if (m->comm_dead) return fail(SLI_ERR_COMM, "the RCCL communicator was aborted by an earlier bounded wait");
     SLI_TRY(bg_sync_tiles(m));
     if (m->exec == SLI_EXEC_PERSIST && !m->graph_exec) SLI_TRY(tpl_prepare(m));
@@ -1394,6 +1420,7 @@ static void destroy(sli_model* m) {
         if (m->pf.graph[b]) (void)hipGraphDestroy(m->pf.graph[b]);
     }
     if (m->comm) ncclCommDestroy(m->comm);
+    hy_destroy(m->bs);
     for (int r = 0; r < sli::kOsMaxRanks; ++r)
         if (m->os_peer[r] && m->os_peer[r] != m->os_buf) (void)hipIpcCloseMemHandle(m->os_peer[r]);
     if (m->os_buf) (void)hipFree(m->os_buf);
@@ -1657,6 +1684,60 @@ int sli_model_create(const sli_model_config* cfg, const void* comm_id, sli_model
     return create_model(cfg, comm_id, nullptr, out);
 }
 
+int sli_stack_create(const sli_stack_config* cfg, sli_model** out) {
+    SLI_CHECK(cfg && out, SLI_ERR_ARG, "sli_stack_create: null");
+    SLI_CHECK(cfg->vocab > 0 && cfg->width > 0 && cfg->max_len > 0 && cfg->batch > 0, SLI_ERR_SHAPE,
+              "sli_stack_create: non-positive dimension");
+    SLI_CHECK(cfg->batch <= 64, SLI_ERR_SHAPE, "sli_stack_create: batch must be at most 64");
+    SLI_HIP(hipSetDevice(cfg->device));
+    sli_model* m = new sli_model();
+    auto bail = [&](int rc) {
+        destroy(m);
+        return rc;
+    };
+    m->c.vocab = cfg->vocab;
+    m->c.dim = cfg->width;
+    m->c.max_len = cfg->max_len;
+    m->c.eps = cfg->eps;
+    m->c.w_dtype = cfg->w_dtype;
+    m->c.kv_dtype = cfg->w_dtype;
+    m->c.tp_size = 1;
+    m->c.device = cfg->device;
+    m->c.batch = cfg->batch;
+    m->B = cfg->batch;
+    m->D = cfg->width;
+    m->T = cfg->max_len;
+    m->V = m->v_n = cfg->vocab;
+    if (hipStreamCreateWithFlags(&m->stream, hipStreamNonBlocking) != hipSuccess)
+        return bail(fail(SLI_ERR_HIP, "hipStreamCreate"));
+    int rc = hy_create(cfg, m->stream, &m->bs);
+    if (rc != SLI_OK) return bail(rc);
+    m->c.n_layers = m->L = hy_runs(m->bs);
+    m->key_ld = hy_key_ld(m->bs, m->B);
+    auto A = [&](void** p, size_t bytes) {
+        if (rc == SLI_OK) rc = model_alloc(m, p, bytes);
+        if (rc == SLI_OK && hipMemset(*p, 0, bytes) != hipSuccess) rc = fail(SLI_ERR_HIP, "memset");
+    };
+    A((void**)&m->logits, sizeof(float) * (size_t)m->B * m->v_n);
+    A((void**)&m->keys, sizeof(unsigned long long) * m->B * m->key_ld);
+    A((void**)&m->bkeys, sizeof(unsigned long long) * m->B);
+    A((void**)&m->st, sizeof(DevState) * m->B);
+    A((void**)&m->prompt, sizeof(int32_t) * m->B * (m->T + 1));
+    A((void**)&m->hist, sizeof(int32_t) * m->B * (m->T + 1));
+    if (rc != SLI_OK || (rc = sli_model_reset(m)) != SLI_OK) return bail(rc);
+    *out = m;
+    return SLI_OK;
+}
+
+int sli_stack_set_tensor(sli_model* m, const char* name, const float* host, int64_t n) {
+    SLI_CHECK(m && name && host, SLI_ERR_ARG, "null argument");
+    SLI_CHECK(m->bs, SLI_ERR_STATE, "not a block-stack model");
+    SLI_HIP(hipSetDevice(m->c.device));
+    return hy_set_tensor(m->bs, name, host, n);
+}
+
+int sli_stack_runs(const sli_model* m) { return m && m->bs ? hy_runs(m->bs) : 0; }
+
 int sli_model_destroy(sli_model* m) {
     SLI_CHECK(!m || !m->group, SLI_ERR_STATE, "a rank of an in-process tp group is destroyed with its group");
     destroy(m);
@@ -1666,6 +1747,7 @@ int sli_model_destroy(sli_model* m) {
 int sli_model_init_synthetic(sli_model* m, uint32_t seed) {
     SLI_CHECK(m, SLI_ERR_ARG, "null model");
     SLI_HIP(hipSetDevice(m->c.device));
+    if (m->bs) return hy_init_synthetic(m->bs, seed);
     auto src = [&](int kind, int index) {
         return SrcSynth{seed, sli_stream_id((uint32_t)kind, (uint32_t)index), synth_c(m, kind),
                         kind == SLI_T_NORM ? 1.0f : 0.0f};
@@ -1681,6 +1763,7 @@ int sli_model_init_synthetic(sli_model* m, uint32_t seed) {
 
 int sli_model_set_weight(sli_model* m, int32_t kind, int32_t index, const float* host, int64_t n) {
     SLI_CHECK(m && host, SLI_ERR_ARG, "null argument");
+    SLI_CHECK(!m->bs, SLI_ERR_STATE, "a block-stack model's tensors go through sli_stack_set_tensor");
     const int64_t want = tensor_elems(m, kind);
     SLI_CHECK(want > 0, SLI_ERR_ARG, "unknown tensor kind");
     SLI_CHECK(n == want, SLI_ERR_SHAPE, "tensor element count does not match the config");
@@ -1698,6 +1781,7 @@ int sli_model_set_weight(sli_model* m, int32_t kind, int32_t index, const float*
 
 int sli_model_load_flat(sli_model* m, const char* path) {
     SLI_CHECK(m && path, SLI_ERR_ARG, "null argument");
+    SLI_CHECK(!m->bs, SLI_ERR_STATE, "a block-stack model's tensors go through sli_stack_set_tensor");
     const int fd = open(path, O_RDONLY);
     SLI_CHECK(fd >= 0, SLI_ERR_ARG, std::string("Fail to open the weight file: ") + path);
     struct stat sb;
@@ -1732,9 +1816,11 @@ int sli_model_load_flat(sli_model* m, const char* path) {
 int sli_model_reset(sli_model* m) {
     SLI_CHECK(m, SLI_ERR_ARG, "null model");
     SLI_HIP(hipSetDevice(m->c.device));
-    const size_t kv = (size_t)m->L * m->B * m->hkv * m->T * m->hd * m->kvbytes;
-    SLI_HIP(hipMemsetAsync(m->kc, 0, kv, m->stream));
-    SLI_HIP(hipMemsetAsync(m->vc, 0, kv, m->stream));
+    if (!m->bs) {  // (a block-stack slot's cache and state start over at position 0 by themselves)
+        const size_t kv = (size_t)m->L * m->B * m->hkv * m->T * m->hd * m->kvbytes;
+        SLI_HIP(hipMemsetAsync(m->kc, 0, kv, m->stream));
+        SLI_HIP(hipMemsetAsync(m->vc, 0, kv, m->stream));
+    }
     std::vector<DevState> h(m->B);
     for (auto& d : h) d.advance = 1;
     return upload_states(m, h);
@@ -1745,7 +1831,7 @@ int sli_model_fill_kv_synthetic(sli_model* m, uint32_t seed, int32_t upto) {
     SLI_CHECK(upto >= 0 && upto <= m->T, SLI_ERR_RANGE, "upto out of range");
     if (upto == 0) return SLI_OK;
     SLI_HIP(hipSetDevice(m->c.device));
-    SLI_TRY(SLI_DISPATCH(m, fill_kv, m, seed, upto));
+    SLI_TRY(m->bs ? hy_fill_context(m->bs, seed, upto) : SLI_DISPATCH(m, fill_kv, m, seed, upto));
     SLI_TRY(wait_stream(m));
     return SLI_OK;
 }
@@ -1850,13 +1936,118 @@ static std::vector<PfState> pf_chunks(int n) {
     return cs;
 }
 
-extern "C" int sli_model_prefill_path(const sli_model* m) { return m && m->B == 1 && pf_supported(m) ? 1 : 0; }
+extern "C" int sli_model_prefill_path(const sli_model* m) { return m && m->bs ? 1 : m && m->B == 1 && pf_supported(m) ? 1 : 0; }
 
 extern "C" int sli_model_fused_qkv_attn(sli_model* m) {
-    if (!m || m->B != 1) return 0;
+    if (!m || m->B != 1 || m->bs) return 0;
     int done = 0;
     if (SLI_DISPATCH(m, gemv_qkv_attn, m, 0, &done, true) != SLI_OK) return 0;
     return done;
+}
+
+// The next tokens of n sequences as one batch (sli.h). One token each: a decode pass over n rows. Otherwise the
+// portions are packed into passes of at most kHyMaxRows rows, each portion from a row that is a multiple of kHyTile on
+// (a portion longer than what is left of a pass goes on in the next one from the caches and states it left).
+extern "C" int sli_model_feed(sli_model* m, int32_t n, const int32_t* slots, const int32_t* starts, const int32_t* lens,
+                              const int32_t* tokens, const int32_t* want_n, const int32_t* want, float* logits,
+                              float* hidden) {
+    SLI_CHECK(m && slots && starts && lens && tokens && n >= 1, SLI_ERR_ARG, "null argument");
+    SLI_CHECK(m->bs, SLI_ERR_STATE, "feed: block-stack models only");
+    SLI_HIP(hipSetDevice(m->c.device));
+    SLI_TRY(hy_prepare(m->bs));
+    std::vector<char> used(m->B, 0);
+    std::vector<int64_t> tok0(n), want0(n);
+    int64_t nt = 0, nw = 0;
+    bool one = true;
+    for (int i = 0; i < n; ++i) {
+        SLI_CHECK(slots[i] >= 0 && slots[i] < m->B && !used[slots[i]], SLI_ERR_RANGE, "feed: bad slot");
+        used[slots[i]] = 1;
+        SLI_CHECK(starts[i] >= 0 && lens[i] >= 1 && (int64_t)starts[i] + lens[i] <= m->T, SLI_ERR_RANGE,
+                  "feed: positions out of range");
+        tok0[i] = nt;
+        want0[i] = nw;
+        nt += lens[i];
+        const int wn = want_n ? want_n[i] : 0;
+        SLI_CHECK(wn >= 0 && (wn == 0 || (want && logits)), SLI_ERR_ARG, "feed: logits wanted without a place for them");
+        for (int j = 0; j < wn; ++j)
+            SLI_CHECK(want[nw + j] >= 0 && want[nw + j] < lens[i] && (j == 0 || want[nw + j] > want[nw + j - 1]),
+                      SLI_ERR_RANGE, "feed: wanted places must be ascending places of the entry");
+        nw += wn;
+        one = one && lens[i] == 1;
+    }
+    for (int64_t t = 0; t < nt; ++t)
+        SLI_CHECK(tokens[t] >= 0 && tokens[t] < m->V, SLI_ERR_RANGE, "Token index is greater than vocab size.");
+    const int runs = hy_runs(m->bs);
+    std::vector<int> done(n, 0);
+    std::vector<int32_t> wdone(n, 0);
+    std::vector<float> lbuf, hbuf;
+    int i0 = 0;  // first entry with tokens left
+    while (i0 < n) {
+        std::vector<RowRef> rows;
+        std::vector<SegRef> segs;
+        std::vector<int32_t> widx;
+        std::vector<int64_t> wdst, hdst;  // where each wanted row's logits / each row's residual goes (-1: padding)
+        for (int i = i0; i < n; ++i) {
+            if (!one) {
+                while (rows.size() % kHyTile) {
+                    rows.push_back(RowRef{-1, 0, 0, 0});
+                    hdst.push_back(-1);
+                }
+            }
+            const int room = kHyMaxRows - (int)rows.size(), c = std::min(room, lens[i] - done[i]);
+            if (c <= 0) break;
+            const int first = (int)rows.size();
+            segs.push_back(SegRef{slots[i], first, c, starts[i] + done[i]});
+            for (int j = 0; j < c; ++j) {
+                rows.push_back(RowRef{slots[i], starts[i] + done[i] + j, tokens[tok0[i] + done[i] + j], first});
+                hdst.push_back(tok0[i] + done[i] + j);
+            }
+            const int wn = want_n ? want_n[i] : 0;
+            while (wdone[i] < wn && want[want0[i] + wdone[i]] < done[i] + c) {
+                widx.push_back(first + want[want0[i] + wdone[i]] - done[i]);
+                wdst.push_back(want0[i] + wdone[i]);
+                ++wdone[i];
+            }
+            done[i] += c;
+        }
+        while (i0 < n && done[i0] == lens[i0]) ++i0;
+        lbuf.resize(widx.size() * (size_t)m->V);
+        if (hidden) hbuf.resize((size_t)runs * rows.size() * m->D);
+        SLI_TRY(hy_pass(m->bs, rows, segs, one, widx, lbuf.data(), hidden ? hbuf.data() : nullptr));
+        for (size_t w = 0; w < widx.size(); ++w)
+            std::memcpy(logits + (size_t)wdst[w] * m->V, lbuf.data() + w * m->V, sizeof(float) * m->V);
+        if (hidden)
+            for (int r = 0; r < runs; ++r)
+                for (size_t j = 0; j < rows.size(); ++j)
+                    if (hdst[j] >= 0)
+                        std::memcpy(hidden + ((size_t)r * nt + hdst[j]) * m->D, hbuf.data() + ((size_t)r * rows.size() + j) * m->D,
+                                    sizeof(float) * m->D);
+    }
+    return SLI_OK;
+}
+
+// Positions 0 .. lens[b] - 2 of every sequence's prompt in packed passes; each state is left at its last prompt token.
+extern "C" int sli_model_prefill_batch(sli_model* m, const int32_t* prompts, const int32_t* lens, int32_t ld) {
+    SLI_CHECK(m && prompts && lens, SLI_ERR_ARG, "null argument");
+    SLI_CHECK(m->bs, SLI_ERR_STATE, "prefill_batch: block-stack models only");
+    std::vector<int32_t> slots, starts, ns, toks;
+    for (int b = 0; b < m->B; ++b) {
+        SLI_CHECK(lens[b] >= 1 && lens[b] <= ld && lens[b] <= m->T, SLI_ERR_RANGE, "prompt length out of range");
+        const int32_t* p = prompts + (size_t)b * ld;
+        SLI_TRY(set_prompt(m, b, p, lens[b]));
+        SLI_HIP(hipMemcpyAsync(m->hist + (size_t)b * (m->T + 1), p, sizeof(int32_t) * lens[b], hipMemcpyHostToDevice,
+                               m->stream));
+        if (lens[b] == 1) continue;
+        slots.push_back(b);
+        starts.push_back(0);
+        ns.push_back(lens[b] - 1);
+        toks.insert(toks.end(), p, p + lens[b] - 1);
+    }
+    if (!slots.empty())
+        SLI_TRY(sli_model_feed(m, (int32_t)slots.size(), slots.data(), starts.data(), ns.data(), toks.data(), nullptr,
+                               nullptr, nullptr, nullptr));
+    for (int b = 0; b < m->B; ++b) SLI_TRY(set_state(m, b, prompts[(size_t)b * ld + lens[b] - 1], lens[b] - 1, 1));
+    return SLI_OK;
 }
 
 extern "C" int sli_model_prefill(sli_model* m, const int32_t* ids, int32_t n) {
@@ -1866,6 +2057,7 @@ extern "C" int sli_model_prefill(sli_model* m, const int32_t* ids, int32_t n) {
     SLI_CHECK(n >= 1 && n <= m->T, SLI_ERR_RANGE, "prompt length out of range");
     for (int i = 0; i < n; ++i)
         SLI_CHECK(ids[i] >= 0 && ids[i] < m->V, SLI_ERR_RANGE, "Token index is greater than vocab size.");
+    if (m->bs) return sli_model_prefill_batch(m, ids, &n, n);
     SLI_HIP(hipSetDevice(m->c.device));
     SLI_TRY(set_prompt(m, 0, ids, n));
     SLI_HIP(hipMemcpyAsync(m->hist, ids, sizeof(int32_t) * n, hipMemcpyHostToDevice, m->stream));
@@ -2080,6 +2272,7 @@ int sli_model_get_kv_seq(sli_model* m, int32_t seq, int32_t layer, int32_t which
 
 int sli_model_get_weight(sli_model* m, int32_t kind, int32_t index, float* host, int64_t n) {
     SLI_CHECK(m && host, SLI_ERR_ARG, "null argument");
+    SLI_CHECK(!m->bs, SLI_ERR_STATE, "not available for block-stack models");
     const void* src = nullptr;
     const float* scale = nullptr;
     int64_t rows = 0, cols = 0;
@@ -2144,6 +2337,14 @@ int sli_model_step_bytes(sli_model* m, double* weight_bytes, double* kv_bytes) {
     SLI_CHECK(m, SLI_ERR_ARG, "null model");
     std::vector<DevState> h;
     SLI_TRY(download_states(m, h));
+    if (m->bs) {
+        double ctx = 0.0, wbytes = 0.0, sbytes = 0.0;
+        for (const DevState& d : h) ctx += d.pos + 1.0;
+        hy_step_bytes(m->bs, m->B, ctx, &wbytes, &sbytes);
+        if (weight_bytes) *weight_bytes = wbytes;
+        if (kv_bytes) *kv_bytes = sbytes;
+        return SLI_OK;
+    }
     const double wb = (double)m->wbytes, D = m->D, hd = m->hd;
     const double per_layer = ((m->hq + 2.0 * m->hkv) * hd * D + D * m->hq * hd + 3.0 * m->Il * D) * wb;
     double w = m->L * per_layer + (double)m->v_n * D * wb;
@@ -2289,6 +2490,7 @@ int sli_model_time_steps(sli_model* m, int32_t iters, double* avg_us) {
 
 int sli_model_time_families(sli_model* m, int32_t iters, double* us, double* bytes, int32_t* launches) {
     SLI_CHECK(m && iters > 0 && us && bytes && launches, SLI_ERR_ARG, "bad argument");
+    SLI_CHECK(!m->bs, SLI_ERR_STATE, "not available for block-stack models");
     SLI_CHECK(!m->group, SLI_ERR_STATE, "time a group's ranks through a standalone model");
     SLI_HIP(hipSetDevice(m->c.device));
     SLI_TRY(bg_sync_tiles(m));
@@ -2367,6 +2569,7 @@ __global__ void __launch_bounds__(1024) stream_read_kernel(const char* a, long l
 
 int sli_model_time_stream(sli_model* m, int32_t iters, double* us) {
     SLI_CHECK(m && iters > 0 && us, SLI_ERR_ARG, "bad argument");
+    SLI_CHECK(!m->bs, SLI_ERR_STATE, "not available for block-stack models");
     SLI_CHECK(!m->group, SLI_ERR_STATE, "time a group's ranks through a standalone model");
     SLI_HIP(hipSetDevice(m->c.device));
     struct Guard {
@@ -2421,6 +2624,7 @@ int sli_model_time_stream(sli_model* m, int32_t iters, double* us) {
 int sli_model_time_gemv(sli_model* m, int32_t iters, double* avg_us, double* bytes_per_launch,
                         int32_t* launches_per_step) {
     SLI_CHECK(m && iters > 0, SLI_ERR_ARG, "bad argument");
+    SLI_CHECK(!m->bs, SLI_ERR_STATE, "not available for block-stack models");
     SLI_HIP(hipSetDevice(m->c.device));
     SLI_TRY(bg_sync_tiles(m));  // the batched launches stream the fragment-layout copies
     // The probe re-runs the step's weight-streaming launches in place. It saves and restores the residual

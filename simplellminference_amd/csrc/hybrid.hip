@@ -1,0 +1,686 @@
+// hybrid.hip — block-stack models (hybrid.h): configuration checks, weight placement, caches and states, and the
+// recorded launches of a decode step and of a prompt pass.
+#include "hybrid.h"
+
+#include <algorithm>
+#include <cmath>
+#include <cstdlib>
+#include <cstring>
+#include <map>
+#include <type_traits>
+
+#include "../../include/sli_synth.h"
+#include "attn_rows.h"
+#include "canon.h"
+#include "hybrid_kernels.h"
+#include "retention.h"
+
+namespace sli {
+
+#define HY_TRY(expr)                   \
+    do {                               \
+        int rc_ = (expr);              \
+        if (rc_ != SLI_OK) return rc_; \
+    } while (0)
+
+static int pad_to(int n, int m) { return (n + m - 1) / m * m; }
+
+struct HyLayer {
+    sli_block_desc d{};
+    int mixw = 0, KA = 0, KF = 0, Kp = 0;  // output projection input: [mixer (KA) ; feed-forward (KF)]
+    int hpq = 0, hpv = 0, e_q = 0, e_k = 0, e_v = 0, e_g = 0, u1p = 0, u2p = 0;
+    int hd = 0;   // attention: padded cache row
+    int nsl = 0;  // retention: state slices per head
+    int rot = -1;
+    void *win = nullptr, *wout = nullptr;
+    float *f1 = nullptr, *f2 = nullptr, *r1 = nullptr, *r2 = nullptr, *sink = nullptr, *decay = nullptr;
+    // the output projection's input and the attention query rows, one buffer per shape: their padding columns are never
+    // written, so they stay zero
+    float *cat32 = nullptr, *q = nullptr;
+    __half* cat16 = nullptr;
+    float n1 = 0.0f, n2 = 0.0f;
+    std::vector<float> c1, c2;  // [width][taps] as given
+};
+
+struct HyRun {
+    int layer = 0;
+    void *kc = nullptr, *vc = nullptr;
+    float *S = nullptr, *ring = nullptr;
+};
+
+struct HyRot {
+    int dims = 0;
+    double base = 0.0;
+    float *cs = nullptr, *sn = nullptr;
+};
+
+struct BlockStack {
+    sli_stack_config c{};
+    hipStream_t stream = nullptr;
+    bool f16 = true;
+    size_t wb = 2;
+    int D = 0, Dp = 0, V = 0, Vp = 0, T = 0, B = 0, taps = 0, M = 0;  // taps: padded tap count; M: rows of a pass
+    std::vector<HyLayer> layers;
+    std::vector<HyRun> runs;
+    std::vector<HyRot> rots;
+    void *emb = nullptr, *head = nullptr;
+    float* fnorm = nullptr;  // final gain per channel
+    float fgain = 0.0f;
+    std::map<std::string, bool> want;  // tensor -> placed
+    bool dirty = true;
+    // activations of a pass
+    RowRef* rows = nullptr;
+    SegRef* segs = nullptr;
+    int32_t *nsegs = nullptr, *widx = nullptr;
+    float *x = nullptr, *q = nullptr, *k = nullptr, *v = nullptr, *g = nullptr, *o = nullptr, *lg = nullptr;
+    void *c1 = nullptr, *c2 = nullptr, *xl = nullptr;  // fp32 or fp16 by path
+    std::vector<void*> allocs;
+    std::vector<std::pair<hipGraph_t, hipGraphExec_t>> graphs_one, graphs_rows;
+};
+
+// ---------------------------------------------------------------- creation
+static int hy_alloc(BlockStack* s, void** p, size_t bytes, bool zero = true) {
+    bytes = std::max<size_t>(bytes, 16);
+    hipError_t e = hipMalloc(p, bytes);
+    if (e != hipSuccess) return hip_fail(e, "hipMalloc");
+    s->allocs.push_back(*p);
+    if (zero) SLI_HIP(hipMemset(*p, 0, bytes));
+    return SLI_OK;
+}
+
+static int hy_layer_init(HyLayer& l, int i) {
+    const sli_block_desc& d = l.d;
+    const std::string at = "block " + std::to_string(i) + ": ";
+    SLI_CHECK(d.heads > 0 && d.dim > 0 && d.vdim > 0 && d.ff >= 0, SLI_ERR_SHAPE, at + "non-positive size");
+    SLI_CHECK(d.mixer == SLI_MIX_ATTENTION || d.mixer == SLI_MIX_RETENTION, SLI_ERR_ARG, at + "unknown mixer");
+    l.mixw = d.heads * d.vdim;
+    l.KA = pad_to(l.mixw, 64);
+    l.KF = pad_to(d.ff, 64);
+    l.Kp = l.KA + l.KF;
+    l.hpq = (d.dim + 1) / 2;
+    l.hpv = (d.vdim + 1) / 2;
+    if (d.mixer == SLI_MIX_ATTENTION) {
+        SLI_CHECK(d.kv_heads > 0 && d.heads % d.kv_heads == 0, SLI_ERR_SHAPE, at + "heads must be a multiple of kv_heads");
+        SLI_CHECK(d.vdim <= kAttnRowsMaxV, SLI_ERR_SHAPE, at + "attention vdim must be at most 512");
+        SLI_CHECK(d.dim <= 4096, SLI_ERR_SHAPE, at + "attention dim must be at most 4096");
+        const int w = std::max(d.dim, d.vdim);
+        l.hd = w <= 64 ? 64 : w <= 128 ? 128 : pad_to(w, 64);
+        l.e_q = d.heads * l.hpq;
+        l.e_k = l.e_q + d.kv_heads * l.hpq;
+        l.e_v = l.e_k + d.kv_heads * l.hpv;
+        l.e_g = l.e_v;
+    } else {
+        SLI_CHECK(d.rot_dims >= 0 && d.rot_dims % 2 == 0 && d.rot_dims <= d.dim, SLI_ERR_SHAPE, at + "bad rot_dims");
+        SLI_CHECK(ret_scan_lds(d.dim) <= 160 * 1024, SLI_ERR_SHAPE, at + "retention dim too large");
+        if (ret_scan_lds(d.dim) > 64 * 1024)
+            SLI_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&ret_scan_kernel),
+                                        hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024));
+        l.nsl = (d.vdim + kRetCols - 1) / kRetCols;
+        l.e_q = d.heads * l.hpq;
+        l.e_k = l.e_q + d.heads * l.hpq;
+        l.e_v = l.e_k + d.heads * l.hpv;
+        l.e_g = l.e_v + d.heads * l.hpv;
+    }
+    l.u1p = pad_to(l.e_g, 64);  // 128 rows: a GEMM row block never straddles the two inputs
+    l.u2p = pad_to(d.ff, 64);
+    return SLI_OK;
+}
+
+int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out) {
+    const sli_stack_config& c = *cfg;
+    SLI_CHECK(c.vocab > 0 && c.width > 0 && c.n_blocks > 0 && c.blocks && c.max_len > 0 && c.batch > 0, SLI_ERR_SHAPE,
+              "stack: non-positive dimension");
+    SLI_CHECK(c.taps >= 1 && c.taps <= kCanonMaxTaps, SLI_ERR_SHAPE, "stack: taps must be 1 .. 32");
+    SLI_CHECK(c.loop_start >= 0 && c.loop_start <= c.loop_stop && c.loop_stop <= c.n_blocks && c.loop_times >= 1,
+              SLI_ERR_SHAPE, "stack: bad loop");
+    SLI_CHECK(c.w_dtype == SLI_DT_F16 || c.w_dtype == SLI_DT_F32, SLI_ERR_ARG, "stack: fp16 or fp32 weights");
+    BlockStack* s = new BlockStack();
+    *out = s;  // destroyed by the caller on failure
+    s->c = c;
+    s->stream = stream;
+    s->f16 = c.w_dtype == SLI_DT_F16;
+    s->wb = s->f16 ? 2 : 4;
+    s->D = c.width;
+    s->Dp = pad_to(c.width, 64);
+    s->V = c.vocab;
+    s->Vp = pad_to(c.vocab, 128);
+    s->T = c.max_len;
+    s->B = c.batch;
+    s->taps = std::max(c.taps, kCanonFusedTaps);
+    s->M = kHyMaxRows;
+    s->layers.resize(c.n_blocks);
+    size_t nq = 0, nk = 0, nv = 0, no = 0;
+    int dec = 0;
+    std::map<std::pair<int, int>, HyLayer*> by_out;             // (mixer width, ff)
+    std::map<std::pair<std::pair<int, int>, int>, float*> by_q;  // (heads, dim), padded row
+    for (int i = 0; i < c.n_blocks; ++i) {
+        HyLayer& l = s->layers[i];
+        l.d = c.blocks[i];
+        HY_TRY(hy_layer_init(l, i));
+        const bool att = l.d.mixer == SLI_MIX_ATTENTION;
+        HY_TRY(hy_alloc(s, &l.win, s->wb * (size_t)2 * (l.u1p + l.u2p) * s->Dp));
+        HY_TRY(hy_alloc(s, &l.wout, s->wb * (size_t)pad_to(s->D, 128) * l.Kp));
+        const std::string p = "l" + std::to_string(i) + ".";
+        for (const char* n : {"norm1", "canon1", "mix.q", "mix.k", "mix.v", "mix.o"}) s->want[p + n] = false;
+        HY_TRY(hy_alloc(s, (void**)&l.f1, sizeof(float) * s->taps * s->Dp));
+        if (att) {
+            for (const char* n : {"mix.r1", "mix.r2", "mix.sink"}) s->want[p + n] = false;
+            HY_TRY(hy_alloc(s, (void**)&l.r1, sizeof(float) * l.d.heads));
+            HY_TRY(hy_alloc(s, (void**)&l.r2, sizeof(float) * l.d.heads));
+            HY_TRY(hy_alloc(s, (void**)&l.sink, sizeof(float) * l.d.heads));
+            float*& qb = by_q[{{l.d.heads, l.d.dim}, l.hd}];
+            if (!qb) HY_TRY(hy_alloc(s, (void**)&qb, sizeof(float) * (size_t)s->M * l.d.heads * l.hd));
+            l.q = qb;
+        } else {
+            s->want[p + "mix.g"] = false;
+            SLI_CHECK(c.decay, SLI_ERR_ARG, "stack: retention needs decay values");
+            HY_TRY(hy_alloc(s, (void**)&l.decay, sizeof(float) * l.d.heads));
+            SLI_HIP(hipMemcpy(l.decay, c.decay + dec, sizeof(float) * l.d.heads, hipMemcpyHostToDevice));
+            dec += l.d.heads;
+            nq = std::max(nq, (size_t)l.d.heads * l.d.dim);
+            nk = std::max(nk, (size_t)l.d.heads * l.d.dim);
+            nv = std::max(nv, (size_t)l.mixw);
+            if (l.d.rot_dims > 0) {
+                for (size_t r = 0; r < s->rots.size(); ++r)
+                    if (s->rots[r].dims == l.d.rot_dims && s->rots[r].base == l.d.rot_base) l.rot = (int)r;
+                if (l.rot < 0) {
+                    l.rot = (int)s->rots.size();
+                    HyRot rt;
+                    rt.dims = l.d.rot_dims;
+                    rt.base = l.d.rot_base;
+                    s->rots.push_back(rt);
+                }
+            }
+        }
+        if (l.d.ff > 0) {
+            for (const char* n : {"norm2", "canon2", "mlp.gate", "mlp.up", "mlp.down"}) s->want[p + n] = false;
+            HY_TRY(hy_alloc(s, (void**)&l.f2, sizeof(float) * s->taps * s->Dp));
+        }
+        HyLayer*& same = by_out[{l.mixw, l.d.ff}];
+        if (same) {
+            l.cat32 = same->cat32, l.cat16 = same->cat16;
+        } else {
+            HY_TRY(hy_alloc(s, (void**)&l.cat32, sizeof(float) * (size_t)s->M * l.Kp));
+            if (s->f16) HY_TRY(hy_alloc(s, (void**)&l.cat16, sizeof(__half) * (size_t)s->M * l.Kp));
+            same = &l;
+        }
+        no = std::max(no, (size_t)l.mixw);
+    }
+    for (HyRot& r : s->rots) {  // angles in double, the table in fp32
+        const int h = r.dims / 2;
+        std::vector<float> cs((size_t)s->T * h), sn((size_t)s->T * h);
+        for (int j = 0; j < h; ++j) {
+            const double f = std::pow(r.base, -2.0 * j / r.dims);
+            for (int p = 0; p < s->T; ++p) {
+                cs[(size_t)p * h + j] = (float)std::cos(p * f);
+                sn[(size_t)p * h + j] = (float)std::sin(p * f);
+            }
+        }
+        HY_TRY(hy_alloc(s, (void**)&r.cs, sizeof(float) * cs.size(), false));
+        HY_TRY(hy_alloc(s, (void**)&r.sn, sizeof(float) * sn.size(), false));
+        SLI_HIP(hipMemcpy(r.cs, cs.data(), sizeof(float) * cs.size(), hipMemcpyHostToDevice));
+        SLI_HIP(hipMemcpy(r.sn, sn.data(), sizeof(float) * sn.size(), hipMemcpyHostToDevice));
+    }
+    auto add_run = [&](int i) {
+        HyRun r;
+        r.layer = i;
+        s->runs.push_back(r);
+    };
+    for (int i = 0; i < c.loop_start; ++i) add_run(i);
+    for (int t = 0; t < c.loop_times; ++t)
+        for (int i = c.loop_start; i < c.loop_stop; ++i) add_run(i);
+    for (int i = c.loop_stop; i < c.n_blocks; ++i) add_run(i);
+    for (HyRun& r : s->runs) {
+        const HyLayer& l = s->layers[r.layer];
+        HY_TRY(hy_alloc(s, (void**)&r.ring, sizeof(float) * (size_t)s->B * s->taps * s->Dp));
+        if (l.d.mixer == SLI_MIX_ATTENTION) {
+            const size_t n = (size_t)s->B * l.d.kv_heads * s->T * l.hd * (s->f16 ? 2 : 4);
+            HY_TRY(hy_alloc(s, &r.kc, n));
+            HY_TRY(hy_alloc(s, &r.vc, n));
+        } else {
+            HY_TRY(hy_alloc(s, (void**)&r.S, sizeof(float) * (size_t)s->B * l.d.heads * l.nsl * l.d.dim * kRetCols));
+        }
+    }
+    HY_TRY(hy_alloc(s, &s->emb, s->wb * (size_t)s->V * s->D));
+    HY_TRY(hy_alloc(s, &s->head, s->wb * (size_t)s->Vp * s->Dp));
+    HY_TRY(hy_alloc(s, (void**)&s->fnorm, sizeof(float) * s->Dp));
+    for (const char* n : {"embed", "head", "final.norm"}) s->want[n] = false;
+    const size_t M = s->M;
+    HY_TRY(hy_alloc(s, (void**)&s->rows, sizeof(RowRef) * M));
+    HY_TRY(hy_alloc(s, (void**)&s->segs, sizeof(SegRef) * M));
+    HY_TRY(hy_alloc(s, (void**)&s->nsegs, sizeof(int32_t)));
+    HY_TRY(hy_alloc(s, (void**)&s->widx, sizeof(int32_t) * M));
+    HY_TRY(hy_alloc(s, (void**)&s->x, sizeof(float) * M * s->Dp));
+    HY_TRY(hy_alloc(s, &s->c1, sizeof(float) * M * s->Dp));
+    HY_TRY(hy_alloc(s, &s->c2, sizeof(float) * M * s->Dp));
+    HY_TRY(hy_alloc(s, &s->xl, sizeof(float) * M * s->Dp));
+    HY_TRY(hy_alloc(s, (void**)&s->q, sizeof(float) * M * nq));
+    HY_TRY(hy_alloc(s, (void**)&s->k, sizeof(float) * M * nk));
+    HY_TRY(hy_alloc(s, (void**)&s->v, sizeof(float) * M * nv));
+    HY_TRY(hy_alloc(s, (void**)&s->g, sizeof(float) * M * nv));
+    HY_TRY(hy_alloc(s, (void**)&s->o, sizeof(float) * M * no));
+    HY_TRY(hy_alloc(s, (void**)&s->lg, sizeof(float) * M * s->V));
+    return SLI_OK;
+}
+
+void hy_destroy(BlockStack* s) {
+    if (!s) return;
+    for (auto* v : {&s->graphs_one, &s->graphs_rows})
+        for (auto& g : *v) {
+            if (g.second) (void)hipGraphExecDestroy(g.second);
+            if (g.first) (void)hipGraphDestroy(g.first);
+        }
+    for (void* p : s->allocs) (void)hipFree(p);
+    delete s;
+}
+
+int hy_runs(const BlockStack* s) { return (int)s->runs.size(); }
+
+// ---------------------------------------------------------------- weights
+static int hy_place(BlockStack* s, void* dst, int ld, int col0, const std::vector<int32_t>& map, int ncols,
+                    const float* host) {
+    const size_t n = map.size() * (size_t)ncols;
+    float* tmp = nullptr;
+    int32_t* dm = nullptr;
+    int rc = SLI_OK;
+    if (hipMalloc(&tmp, sizeof(float) * n) != hipSuccess || hipMalloc(&dm, sizeof(int32_t) * map.size()) != hipSuccess)
+        rc = fail(SLI_ERR_NOMEM, "weight staging");
+    if (rc == SLI_OK && (hipMemcpy(tmp, host, sizeof(float) * n, hipMemcpyHostToDevice) != hipSuccess ||
+                         hipMemcpy(dm, map.data(), sizeof(int32_t) * map.size(), hipMemcpyHostToDevice) != hipSuccess))
+        rc = fail(SLI_ERR_HIP, "weight upload");
+    if (rc == SLI_OK) {
+        const dim3 grid((unsigned)map.size());
+        if (s->f16)
+            hipLaunchKernelGGL(hy_place_kernel<__half>, grid, dim3(256), 0, s->stream, (__half*)dst, ld, col0, dm, ncols, tmp);
+        else
+            hipLaunchKernelGGL(hy_place_kernel<float>, grid, dim3(256), 0, s->stream, (float*)dst, ld, col0, dm, ncols, tmp);
+        if (hipGetLastError() != hipSuccess || hipStreamSynchronize(s->stream) != hipSuccess)
+            rc = fail(SLI_ERR_HIP, "weight placement");
+    }
+    if (tmp) (void)hipFree(tmp);
+    if (dm) (void)hipFree(dm);
+    return rc;
+}
+
+// fused-matrix rows of a head-wise tensor: `heads` heads of n dims, rh rotation pairs, from pair u0 on
+static std::vector<int32_t> head_rows(int heads, int n, int rh, int u0) {
+    std::vector<int32_t> map;
+    const int hp = (n + 1) / 2;
+    for (int h = 0; h < heads; ++h)
+        for (int d = 0; d < n; ++d) {
+            const int j = d < rh ? d : d < 2 * rh ? d - rh : d / 2;
+            const int e = d < rh ? 0 : d < 2 * rh ? 1 : d & 1;
+            map.push_back(2 * (u0 + h * hp + j) + e);
+        }
+    return map;
+}
+static std::vector<int32_t> strided_rows(int n, int first, int step) {
+    std::vector<int32_t> map(n);
+    for (int i = 0; i < n; ++i) map[i] = first + step * i;
+    return map;
+}
+
+// shape of a tensor: rows x cols (vectors: 1 x n), 0 rows: unknown name
+static void hy_shape(const BlockStack* s, const std::string& name, int* li, std::string* leaf, int64_t* rows, int64_t* cols) {
+    *li = -1;
+    *rows = *cols = 0;
+    *leaf = name;
+    if (name == "embed" || name == "head") {
+        *rows = s->V, *cols = s->D;
+        return;
+    }
+    if (name == "final.norm") {
+        *rows = *cols = 1;
+        return;
+    }
+    const size_t dot = name.find('.');
+    *li = std::atoi(name.c_str() + 1);
+    *leaf = name.substr(dot + 1);
+    const sli_block_desc& d = s->layers[*li].d;
+    const int kvh = d.mixer == SLI_MIX_ATTENTION ? d.kv_heads : d.heads;
+    const std::string& t = *leaf;
+    auto set = [&](int64_t r, int64_t c) { *rows = r, *cols = c; };
+    if (t == "norm1" || t == "norm2") set(1, 1);
+    else if (t == "canon1" || t == "canon2") set(s->D, s->c.taps);
+    else if (t == "mix.q") set((int64_t)d.heads * d.dim, s->D);
+    else if (t == "mix.k") set((int64_t)kvh * d.dim, s->D);
+    else if (t == "mix.v") set((int64_t)kvh * d.vdim, s->D);
+    else if (t == "mix.g") set((int64_t)d.heads * d.vdim, s->D);
+    else if (t == "mix.o") set(s->D, (int64_t)d.heads * d.vdim);
+    else if (t == "mix.r1" || t == "mix.r2" || t == "mix.sink") set(1, d.heads);
+    else if (t == "mlp.gate" || t == "mlp.up") set(d.ff, s->D);
+    else if (t == "mlp.down") set(s->D, d.ff);
+}
+
+int hy_set_tensor(BlockStack* s, const std::string& name, const float* host, int64_t n) {
+    auto it = s->want.find(name);
+    SLI_CHECK(it != s->want.end(), SLI_ERR_ARG, "the model has no tensor '" + name + "'");
+    int li;
+    std::string t;
+    int64_t rows, cols;
+    hy_shape(s, name, &li, &t, &rows, &cols);
+    SLI_CHECK(n == rows * cols, SLI_ERR_SHAPE, "tensor '" + name + "' has the wrong size");
+    if (s->f16)
+        for (int64_t i = 0; i < n; ++i)
+            SLI_CHECK(std::fabs(host[i]) <= 65504.0f, SLI_ERR_RANGE, "tensor '" + name + "' has values fp16 cannot hold");
+    s->dirty = true;
+    int rc = SLI_OK;
+    if (name == "embed") {
+        rc = hy_place(s, s->emb, s->D, 0, strided_rows(s->V, 0, 1), s->D, host);
+    } else if (name == "head") {
+        rc = hy_place(s, s->head, s->Dp, 0, strided_rows(s->V, 0, 1), s->D, host);
+    } else if (name == "final.norm") {
+        s->fgain = host[0];
+    } else {
+        HyLayer& l = s->layers[li];
+        const sli_block_desc& d = l.d;
+        const int kvh = d.mixer == SLI_MIX_ATTENTION ? d.kv_heads : d.heads;
+        const int rh = d.mixer == SLI_MIX_RETENTION ? d.rot_dims / 2 : 0;
+        if (t == "norm1") l.n1 = host[0];
+        else if (t == "norm2") l.n2 = host[0];
+        else if (t == "canon1") l.c1.assign(host, host + n);
+        else if (t == "canon2") l.c2.assign(host, host + n);
+        else if (t == "mix.q") rc = hy_place(s, l.win, s->Dp, 0, head_rows(d.heads, d.dim, rh, 0), s->D, host);
+        else if (t == "mix.k") rc = hy_place(s, l.win, s->Dp, 0, head_rows(kvh, d.dim, rh, l.e_q), s->D, host);
+        else if (t == "mix.v") rc = hy_place(s, l.win, s->Dp, 0, head_rows(kvh, d.vdim, 0, l.e_k), s->D, host);
+        else if (t == "mix.g") rc = hy_place(s, l.win, s->Dp, 0, head_rows(d.heads, d.vdim, 0, l.e_v), s->D, host);
+        else if (t == "mix.o") rc = hy_place(s, l.wout, l.Kp, 0, strided_rows(s->D, 0, 1), l.mixw, host);
+        else if (t == "mlp.gate") rc = hy_place(s, l.win, s->Dp, 0, strided_rows(d.ff, 2 * l.u1p, 2), s->D, host);
+        else if (t == "mlp.up") rc = hy_place(s, l.win, s->Dp, 0, strided_rows(d.ff, 2 * l.u1p + 1, 2), s->D, host);
+        else if (t == "mlp.down") rc = hy_place(s, l.wout, l.Kp, l.KA, strided_rows(s->D, 0, 1), d.ff, host);
+        else {
+            float* p = t == "mix.r1" ? l.r1 : t == "mix.r2" ? l.r2 : l.sink;
+            SLI_HIP(hipMemcpy(p, host, sizeof(float) * n, hipMemcpyHostToDevice));
+        }
+    }
+    if (rc == SLI_OK) it->second = true;
+    return rc;
+}
+
+int hy_init_synthetic(BlockStack* s, uint32_t seed) {
+    std::vector<std::string> names;
+    for (auto& kv : s->want) names.push_back(kv.first);
+    std::vector<float> buf, block(1 << 20);
+    uint64_t st = 0x9E3779B97F4A7C15ull * (seed + 1);
+    auto rnd = [&]() {  // xorshift*, uniform in (-1, 1)
+        st ^= st >> 12, st ^= st << 25, st ^= st >> 27;
+        return (float)((double)((st * 0x2545F4914F6CDD1Dull) >> 40) / 8388608.0 - 1.0);
+    };
+    for (float& f : block) f = rnd();
+    for (const std::string& name : names) {
+        int li;
+        std::string t;
+        int64_t rows, cols;
+        hy_shape(s, name, &li, &t, &rows, &cols);
+        const int64_t n = rows * cols;
+        buf.resize(n);
+        const bool gain = t == "norm1" || t == "norm2" || t == "final.norm";
+        const float a = gain ? 0.1f : t == "mix.r2" ? 0.2f : rows == 1 ? 1.0f
+                        : t == "canon1" || t == "canon2" ? 0.3f : t == "embed" ? 1.0f : 1.5f / std::sqrt((float)cols);
+        const float off = gain ? 1.0f : t == "mix.r2" ? 0.25f : rows == 1 ? 1.0f : 0.0f;
+        // one random block, read from a random offset per row (large matrices fill at memory speed)
+        for (int64_t i = 0; i < n;) {
+            st ^= st >> 12, st ^= st << 25, st ^= st >> 27;
+            const size_t o = (size_t)((st * 0x2545F4914F6CDD1Dull) >> 45) & ((1 << 19) - 1);
+            const int64_t c = std::min<int64_t>(std::min<int64_t>(n - i, 1 << 19), std::max<int64_t>(cols, 1));
+            for (int64_t j = 0; j < c; ++j) buf[i + j] = off + a * block[o + j];
+            i += c;
+        }
+        HY_TRY(hy_set_tensor(s, name, buf.data(), n));
+    }
+    return SLI_OK;
+}
+
+int hy_prepare(BlockStack* s) {
+    if (!s->dirty) return SLI_OK;
+    for (auto& kv : s->want) SLI_CHECK(kv.second, SLI_ERR_STATE, "tensor '" + kv.first + "' was not loaded");
+    SLI_HIP(hipStreamSynchronize(s->stream));
+    const int given = s->c.taps, Dp = s->Dp;
+    for (HyLayer& l : s->layers) {
+        auto fold = [&](const std::vector<float>& w, float gain, float* dst) -> int {
+            std::vector<float> f((size_t)s->taps * Dp, 0.0f);
+            for (int d = 0; d < s->D; ++d)
+                for (int j = 0; j < given; ++j) {
+                    const double c = (double)w[(size_t)d * given + given - 1 - j] + (j == 0 ? 1.0 : 0.0);
+                    f[(size_t)j * Dp + d] = (float)(gain * c);
+                }
+            SLI_HIP(hipMemcpy(dst, f.data(), sizeof(float) * f.size(), hipMemcpyHostToDevice));
+            return SLI_OK;
+        };
+        HY_TRY(fold(l.c1, l.n1, l.f1));
+        if (l.d.ff > 0) HY_TRY(fold(l.c2, l.n2, l.f2));
+    }
+    std::vector<float> g(Dp, 0.0f);
+    std::fill(g.begin(), g.begin() + s->D, s->fgain);
+    SLI_HIP(hipMemcpy(s->fnorm, g.data(), sizeof(float) * Dp, hipMemcpyHostToDevice));
+    s->dirty = false;
+    return SLI_OK;
+}
+
+// ---------------------------------------------------------------- the forward pass over rows
+template <typename WT>
+struct HyRec {
+    using KT = WT;  // fp16 weights with an fp16 cache, fp32 with fp32
+    BlockStack* s;
+    int M;      // rows of the launches
+    bool one;   // one row per sequence (decode)
+    int msegs;  // portions at most
+    hipStream_t st() const { return s->stream; }
+
+    template <class Epi>
+    int project(const void* W, const void* X, int K, int npairs, int u0, const Epi& e) const {
+        SLI_HIP((launch_rows_gemm<WT, Epi>((const WT*)W + (size_t)2 * u0 * K, (const float*)X, K, npairs, u0, M, e, st())));
+        return SLI_OK;
+    }
+    template <typename OT>
+    static OT* cat(const HyLayer& l) {
+        if constexpr (std::is_same<OT, float>::value)
+            return l.cat32;
+        else
+            return l.cat16;
+    }
+    CanonArgs canon(const HyLayer& l, const HyRun& r) const {
+        return CanonArgs{s->x, r.ring, l.f1, l.f2, s->rows, s->c.eps, s->D, s->Dp, s->taps, M};
+    }
+    template <typename OT>
+    HyIn<KT, OT> in_epi(const HyLayer& l, const HyRun& r) const {
+        const sli_block_desc& d = l.d;
+        HyIn<KT, OT> e{};
+        e.retention = d.mixer == SLI_MIX_RETENTION;
+        e.H = d.heads, e.G = d.kv_heads, e.dim = d.dim, e.vdim = d.vdim, e.hpq = l.hpq, e.hpv = l.hpv;
+        e.e_q = l.e_q, e.e_k = l.e_k, e.e_v = l.e_v, e.e_g = l.e_g, e.u1p = l.u1p, e.ff = d.ff;
+        e.rh = l.rot >= 0 ? d.rot_dims / 2 : 0;
+        e.hd = l.hd, e.T = s->T;
+        e.kscale = (float)(1.0 / std::sqrt((double)d.dim));
+        e.limit = d.ff_limit;
+        if (l.rot >= 0) e.cs = s->rots[l.rot].cs, e.sn = s->rots[l.rot].sn;
+        e.q = l.q ? l.q : s->q, e.k = s->k, e.v = s->v, e.g = s->g;
+        e.kc = (KT*)r.kc, e.vc = (KT*)r.vc;
+        e.act = cat<OT>(l), e.act_ld = l.Kp, e.act_off = l.KA;
+        e.rows = s->rows;
+        return e;
+    }
+    template <typename OT>
+    int mixer(const HyLayer& l, const HyRun& r) const {
+        const sli_block_desc& d = l.d;
+        if (d.mixer == SLI_MIX_ATTENTION) {
+            AttnRowsArgs a{l.q, r.kc, r.vc, s->rows, l.r1, l.r2, l.sink, d.heads, d.kv_heads, d.dim, d.vdim, l.hd,
+                           s->T, M, d.scale};
+            hipLaunchKernelGGL((attn_rows_kernel<KT, OT>), dim3(d.heads, M), dim3(64), sizeof(float) * (d.dim + 64), st(),
+                               a, cat<OT>(l), l.Kp);
+        } else {
+            RetArgs a{s->q, s->k, s->v, r.S, s->o, l.decay, s->rows, s->segs, s->nsegs, d.heads, d.dim, d.vdim, l.nsl};
+            if (one)
+                hipLaunchKernelGGL(ret_step_kernel, dim3(l.nsl, d.heads, M), dim3(256), 0, st(), a);
+            else
+                hipLaunchKernelGGL(ret_scan_kernel, dim3(l.nsl, d.heads, msegs), dim3(256), ret_scan_lds(d.dim), st(), a);
+            SLI_HIP(hipGetLastError());
+            hipLaunchKernelGGL(ret_gate_kernel<OT>, dim3((M * d.heads + 3) / 4), dim3(256), 0, st(), s->o, s->g, s->rows,
+                               cat<OT>(l), l.Kp, M, d.heads, d.vdim, s->c.eps);
+        }
+        SLI_HIP(hipGetLastError());
+        return SLI_OK;
+    }
+    int layer(const HyRun& r) const {
+        const HyLayer& l = s->layers[r.layer];
+        using OT = float;
+        const CanonArgs ca = canon(l, r);
+        hipLaunchKernelGGL(canon_rows_kernel<OT>, dim3(M), dim3(256), 0, st(), ca, (OT*)s->c1,
+                           l.d.ff > 0 ? (OT*)s->c2 : (OT*)nullptr, one ? 1 : 0);
+        SLI_HIP(hipGetLastError());
+        if (!one) {
+            hipLaunchKernelGGL(canon_ring_kernel, dim3(M), dim3(256), 0, st(), ca);
+            SLI_HIP(hipGetLastError());
+        }
+        const auto ei = in_epi<OT>(l, r);
+        HY_TRY(project(l.win, s->c1, s->Dp, l.e_g, 0, ei));
+        if (l.d.ff > 0) HY_TRY(project(l.win, s->c2, s->Dp, l.d.ff, l.u1p, ei));
+        HY_TRY(mixer<OT>(l, r));
+        const HyOut eo{s->x, s->Dp, s->D, s->c.residual_mult};
+        return project(l.wout, cat<OT>(l), l.Kp, (s->D + 1) / 2, 0, eo);
+    }
+    int embed() const {
+        hipLaunchKernelGGL(hy_embed_kernel<WT>, dim3(M), dim3(256), 0, st(), s->rows, (const WT*)s->emb, s->c.emb_scale,
+                           s->x, s->V, s->D, s->Dp);
+        SLI_HIP(hipGetLastError());
+        return SLI_OK;
+    }
+    // logits [n][V] of rows idx (null: rows 0 .. n - 1)
+    int logits(const int32_t* idx, int n, float* y) const {
+        using OT = float;
+        hipLaunchKernelGGL(norm_rows_kernel<OT>, dim3(n), dim3(256), 0, st(), s->x, idx, s->fnorm, (OT*)s->xl, s->D, s->Dp,
+                           s->c.eps);
+        SLI_HIP(hipGetLastError());
+        HyRec h = *this;
+        h.M = n;
+        return h.project(s->head, s->xl, s->Dp, (s->V + 1) / 2, 0, HyLogits{y, s->V, n});
+    }
+    int pass() const {
+        HY_TRY(embed());
+        for (const HyRun& r : s->runs) HY_TRY(layer(r));
+        return SLI_OK;
+    }
+    int step(const DevState* dst, float* y, unsigned long long* keys, int key_ld, int* nkeys) const {
+        hipLaunchKernelGGL(hy_rows_kernel, dim3(1), dim3(64), 0, st(), dst, s->rows, M);
+        SLI_HIP(hipGetLastError());
+        HY_TRY(pass());
+        HY_TRY(logits(nullptr, M, y));
+        hipLaunchKernelGGL(hy_keys_kernel, dim3(M), dim3(256), 0, st(), y, s->V, keys, key_ld);
+        SLI_HIP(hipGetLastError());
+        *nkeys = 1;
+        return SLI_OK;
+    }
+};
+
+#define HY_DISPATCH(s, M, one, msegs, CALL) \
+    ((s)->f16 ? HyRec<__half>{(s), (M), (one), (msegs)}.CALL : HyRec<float>{(s), (M), (one), (msegs)}.CALL)
+
+int hy_key_ld(const BlockStack*, int) { return std::max(1, gemv_max_blocks()); }
+
+int hy_record_step(BlockStack* s, const DevState* st, int B, float* logits, unsigned long long* keys, int key_ld,
+                   int* nkeys) {
+    return HY_DISPATCH(s, B, true, B, step(st, logits, keys, key_ld, nkeys));
+}
+
+static int hy_capture(BlockStack* s, std::pair<hipGraph_t, hipGraphExec_t>& g, int M, bool one, int msegs) {
+    if (g.second) return SLI_OK;
+    SLI_HIP(hipStreamBeginCapture(s->stream, hipStreamCaptureModeRelaxed));
+    const int rc = HY_DISPATCH(s, M, one, msegs, pass());
+    hipGraph_t gr = nullptr;
+    const hipError_t e = hipStreamEndCapture(s->stream, &gr);
+    if (rc != SLI_OK || e != hipSuccess) {
+        if (gr) (void)hipGraphDestroy(gr);
+        return rc != SLI_OK ? rc : hip_fail(e, "hipStreamEndCapture");
+    }
+    g.first = gr;
+    SLI_HIP(hipGraphInstantiate(&g.second, gr, nullptr, nullptr, 0));
+    return SLI_OK;
+}
+
+int hy_pass(BlockStack* s, const std::vector<RowRef>& rows_in, const std::vector<SegRef>& segs, bool one,
+            const std::vector<int32_t>& want, float* logits_host, float* hidden_host) {
+    const int n = (int)rows_in.size();
+    SLI_CHECK(n >= 1 && n <= s->M && !segs.empty() && (int)segs.size() <= s->M, SLI_ERR_SHAPE, "pass: too many rows");
+    // a decode step runs its rows as they are; a prompt pass is padded to a row count with a captured graph
+    int M = n, gi = n - 1;
+    if (!one) {
+        M = kHyTile, gi = 0;
+        while (M < n) M *= 2, ++gi;
+    }
+    std::vector<RowRef> rows(rows_in);
+    rows.resize(M, RowRef{-1, 0, 0, 0});
+    const int32_t ns = (int32_t)segs.size();
+    SLI_HIP(hipMemcpyAsync(s->rows, rows.data(), sizeof(RowRef) * M, hipMemcpyHostToDevice, s->stream));
+    SLI_HIP(hipMemcpyAsync(s->segs, segs.data(), sizeof(SegRef) * ns, hipMemcpyHostToDevice, s->stream));
+    SLI_HIP(hipMemcpyAsync(s->nsegs, &ns, sizeof(ns), hipMemcpyHostToDevice, s->stream));
+    const int msegs = one ? M : std::min(s->B, M / kHyTile);
+    if (hidden_host) {  // eager, with a copy after every run
+        HY_TRY(HY_DISPATCH(s, M, one, msegs, embed()));
+        for (size_t r = 0; r < s->runs.size(); ++r) {
+            HY_TRY(HY_DISPATCH(s, M, one, msegs, layer(s->runs[r])));
+            SLI_HIP(hipMemcpy2DAsync(hidden_host + r * (size_t)n * s->D, sizeof(float) * s->D, s->x, sizeof(float) * s->Dp,
+                                     sizeof(float) * s->D, n, hipMemcpyDeviceToHost, s->stream));
+        }
+    } else {
+        auto& gs = one ? s->graphs_one : s->graphs_rows;
+        if ((int)gs.size() <= gi) gs.resize(gi + 1, {nullptr, nullptr});
+        SLI_HIP(hipStreamSynchronize(s->stream));
+        HY_TRY(hy_capture(s, gs[gi], M, one, msegs));
+        SLI_HIP(hipGraphLaunch(gs[gi].second, s->stream));
+    }
+    if (!want.empty()) {
+        const int nw = (int)want.size();
+        SLI_HIP(hipMemcpyAsync(s->widx, want.data(), sizeof(int32_t) * nw, hipMemcpyHostToDevice, s->stream));
+        HY_TRY(HY_DISPATCH(s, M, one, msegs, logits(s->widx, nw, s->lg)));
+        SLI_HIP(hipMemcpyAsync(logits_host, s->lg, sizeof(float) * (size_t)nw * s->V, hipMemcpyDeviceToHost, s->stream));
+    }
+    SLI_HIP(hipStreamSynchronize(s->stream));
+    return SLI_OK;
+}
+
+// ---------------------------------------------------------------- bench helpers
+__global__ void hy_fill_kernel(void* p, size_t n, int f16, uint32_t seed) {
+    for (size_t i = blockIdx.x * (size_t)blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
+        uint32_t h = (uint32_t)(i * 2654435761u) ^ seed;
+        h ^= h >> 16, h *= 0x7feb352du, h ^= h >> 15;
+        const float f = (float)(h & 0xFFFF) / 32768.0f - 1.0f;
+        if (f16)
+            ((__half*)p)[i] = __float2half_rn(f);
+        else
+            ((float*)p)[i] = f;
+    }
+}
+
+int hy_fill_context(BlockStack* s, uint32_t seed, int) {
+    for (HyRun& r : s->runs) {
+        const HyLayer& l = s->layers[r.layer];
+        auto fill = [&](void* p, size_t n, int f16) {
+            if (p) hipLaunchKernelGGL(hy_fill_kernel, dim3(1024), dim3(256), 0, s->stream, p, n, f16, seed);
+        };
+        fill(r.ring, (size_t)s->B * s->taps * s->Dp, 0);
+        fill(r.S, (size_t)s->B * l.d.heads * l.nsl * l.d.dim * kRetCols, 0);
+        const size_t n = (size_t)s->B * l.d.kv_heads * s->T * l.hd;
+        fill(r.kc, n, s->f16);
+        fill(r.vc, n, s->f16);
+        SLI_HIP(hipGetLastError());
+    }
+    return SLI_OK;
+}
+
+void hy_step_bytes(const BlockStack* s, int B, double pos_sum, double* weight_bytes, double* state_bytes) {
+    double w = (double)s->V * s->D * s->wb, k = 0.0;
+    for (const HyRun& r : s->runs) {
+        const HyLayer& l = s->layers[r.layer];
+        const sli_block_desc& d = l.d;
+        w += s->wb * (2.0 * (l.e_g + d.ff) * s->D + (double)s->D * (l.mixw + d.ff));
+        k += 4.0 * B * s->taps * s->D;
+        if (d.mixer == SLI_MIX_ATTENTION)
+            k += pos_sum * d.kv_heads * (d.dim + d.vdim) * (s->f16 ? 2 : 4);
+        else
+            k += 2.0 * 4.0 * B * d.heads * d.dim * d.vdim;
+    }
+    *weight_bytes = w;
+    *state_bytes = k;
+}
+
+}  // namespace sli

@@ -16,6 +16,17 @@ struct DevState {
     unsigned long long key;  // argmax key of the last step (0 between steps)
 };
 
+// One row of a packed forward pass over several sequences (hybrid.h): the sequence slot whose cache and state the
+// row's token uses, its position, and the first row of its portion in the pass (a portion's rows are consecutive,
+// at consecutive positions). slot < 0: padding.
+struct RowRef {
+    int32_t slot, pos, tok, first;
+};
+// A portion: n rows of one sequence from row0 on, the first at position pos0.
+struct SegRef {
+    int32_t slot, row0, n, pos0;
+};
+
 // model.cpp:157-183: next position; teacher-forced prompt token while inside the prompt, else greedy.
 __device__ __forceinline__ void finalize_state(DevState* st, const int32_t* prompt, int32_t* hist, int T) {
     const unsigned long long k = st->key;
