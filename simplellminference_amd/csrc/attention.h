@@ -48,6 +48,10 @@ struct AttnArgs {
     unsigned* hand_count = nullptr;  // attn_hand_bytes: q/k/v units landed per kv head (kAttnHandSub counters, one
                                      // per 128-byte line), then live workgroups done per kv head (the last resets)
     unsigned hand_expect = 0;        // units per kv head: (G + 2) * hd / 2
+    // packed rows (attn_mfma.h ROWS): sequence i of the launch uses cache slot slot_dev[i * pos_seq_stride] (< 0: none),
+    // with a distance bias r1 ln(1 + r2 distance) per query head of a sequence
+    const int32_t* slot_dev = nullptr;
+    const float *bias_r1 = nullptr, *bias_r2 = nullptr;
     int* hand_err = nullptr;         // DevState::error: a bounded wait that gave up sets kAttnErrHand
 };
 

@@ -177,7 +177,9 @@ __device__ __forceinline__ void am_merge(const float* part, float* out, int kvh,
 // grid: n_kv_heads (every sequence's) * max_splits workgroups of 256 threads; a.ppwg = kAmWgKeys * tpw (the
 // split length), NBUF = min(tpw, 2) ring slots per wave. The K/V rows of a split are read once (clamped to pos:
 // rows past the live context re-read row pos, an L2 hit, and are masked).
-template <int HD, int G, int NBUF>
+// ROWS: packed rows (AttnArgs slot_dev, the distance bias); the split partials are always left to a merge that adds
+// the sink (attn_rows.h attn_sink_merge_kernel).
+template <int HD, int G, int NBUF, bool ROWS = false>
 __global__ void __launch_bounds__(64 * kAmWaves) attn_mfma_kernel(AttnArgs<__half> a) {
     using Geo = AmGeo<HD, G>;
     constexpr int ND = Geo::ND, NT = Geo::NT, P = Geo::PIECES;
@@ -201,7 +203,18 @@ __global__ void __launch_bounds__(64 * kAmWaves) attn_mfma_kernel(AttnArgs<__hal
     char* wimg = sm + wave * WB;
     const unsigned wbase = (unsigned)(uintptr_t)(const __attribute__((address_space(3))) char*)wimg;
     const unsigned qbase = wbase, tbase = wbase + Geo::QB;
-    const int ch = a.cache_heads > 0 ? kvh % a.cache_heads : kvh / a.kv_group;
+    int ch = a.cache_heads > 0 ? kvh % a.cache_heads : kvh / a.kv_group;
+    float bias1 = 0.0f, bias2 = 0.0f;
+    if constexpr (ROWS) {
+        const int seq = kvh / a.seq_heads, hs = kvh - seq * a.seq_heads;
+        const int slot = a.slot_dev[(size_t)seq * a.pos_seq_stride];
+        if (slot < 0) return;
+        ch = slot * (a.seq_heads / a.kv_group) + hs / a.kv_group;
+        const int qhead = hs * G + min(i16, G - 1);
+        bias1 = a.bias_r1[qhead];
+        bias2 = a.bias_r2[qhead];
+        asm volatile("" : "+v"(bias1), "+v"(bias2));  // landed before the first DMA piece (counted vmcnt from there on)
+    }
     const __half* kc = a.k + (long long)ch * a.head_stride;
     const __half* vc = a.v + (long long)ch * a.head_stride;
 
@@ -307,7 +320,9 @@ __global__ void __launch_bounds__(64 * kAmWaves) attn_mfma_kernel(AttnArgs<__hal
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int key = t0 + kt * 16 + 4 * g + r;
-                const float v = key <= pos ? sacc[kt][r] * a.scale : -INFINITY;
+                float sc = sacc[kt][r] * a.scale;
+                if constexpr (ROWS) sc -= bias1 * __logf(1.0f + bias2 * (float)(pos - key));
+                const float v = key <= pos ? sc : -INFINITY;
                 sv[kt * 4 + r] = v;
                 cmax = fmaxf(cmax, v);
             }
@@ -381,7 +396,7 @@ __global__ void __launch_bounds__(64 * kAmWaves) attn_mfma_kernel(AttnArgs<__hal
         w4[w] = m4[w] == -INFINITY ? 0.0f : expf(m4[w] - M);
         L = fmaf(w4[w], reinterpret_cast<const float*>(sm + w * WB)[NT * 256 + 64 + lane], L);
     }
-    const bool publish = a.defer_merge == 0;
+    const bool publish = !ROWS && a.defer_merge == 0;
     for (int t = wave; t < NT; t += kAmWaves) {
         am_float4 acc = am_float4{0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll

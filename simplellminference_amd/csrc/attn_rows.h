@@ -76,4 +76,27 @@ __global__ void __launch_bounds__(64) attn_rows_kernel(AttnRowsArgs a, OT* out, 
     }
 }
 
+// Merge of split partials [M H][max_splits][hd + pad] (o, m, l: attn_mfma.h) with the sink: row m's live splits are
+// those that start at or before its position. grid (H, M), 128 threads, one value dim each.
+template <typename OT>
+__global__ void __launch_bounds__(128) attn_sink_merge_kernel(const float* __restrict__ part, AttnRowsArgs a, int max_splits,
+                                                              int ppwg, OT* out, int ldo) {
+    const int h = blockIdx.x, m = blockIdx.y;
+    const RowRef r = a.rows[m];
+    if (r.slot < 0) return;
+    const int ns = min(r.pos / ppwg + 1, max_splits), ps = a.hd + kAttnPartPad;
+    const float* p = part + (size_t)(m * a.H + h) * max_splits * ps;
+    float M = a.sink[h];
+    for (int s = 0; s < ns; ++s) M = fmaxf(M, p[(size_t)s * ps + a.hd]);
+    for (int d = threadIdx.x; d < a.vdim; d += 128) {
+        float o = 0.0f, L = expf(a.sink[h] - M);
+        for (int s = 0; s < ns; ++s) {
+            const float w = expf(p[(size_t)s * ps + a.hd] - M);
+            o = fmaf(w, p[(size_t)s * ps + d], o);
+            L = fmaf(w, p[(size_t)s * ps + a.hd + 1], L);
+        }
+        out[(size_t)m * ldo + (size_t)h * a.vdim + d] = from_f32<OT>(o / L);
+    }
+}
+
 }  // namespace sli

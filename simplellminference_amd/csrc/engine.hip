@@ -1115,9 +1115,9 @@ struct StepRecorder {
             if constexpr (std::is_same<KT, __half>::value) {  // MFMA, 16 chunk rows per workgroup
                 const dim3 ag(M / 16, m->hq);
                 if (hd == 128)
-                    hipLaunchKernelGGL((pf_attn_mfma_kernel<128>), ag, dim3(256), 0, s, aa, f.ps);
+                    hipLaunchKernelGGL((pf_attn_mfma_kernel<128>), ag, dim3(256), 0, s, aa, f.ps, PfRowsArgs{});
                 else
-                    hipLaunchKernelGGL((pf_attn_mfma_kernel<64>), ag, dim3(256), 0, s, aa, f.ps);
+                    hipLaunchKernelGGL((pf_attn_mfma_kernel<64>), ag, dim3(256), 0, s, aa, f.ps, PfRowsArgs{});
             } else {  // fp32 cache: fp32 VALU, 64 chunk rows per workgroup
                 const dim3 ag((M + kPaQB - 1) / kPaQB, m->hq);
                 if (hd == 128)

@@ -10,10 +10,12 @@
 #include <type_traits>
 
 #include "../../include/sli_synth.h"
+#include "attn_mfma.h"
 #include "attn_rows.h"
 #include "canon.h"
 #include "hybrid_kernels.h"
 #include "retention.h"
+#include "retention_chunk.h"
 
 namespace sli {
 
@@ -22,6 +24,8 @@ namespace sli {
         int rc_ = (expr);              \
         if (rc_ != SLI_OK) return rc_; \
     } while (0)
+
+constexpr int kHySection = 128;  // pairs: a GEMM row block (at most 256 rows) never straddles the two inputs
 
 static int pad_to(int n, int m) { return (n + m - 1) / m * m; }
 
@@ -64,7 +68,7 @@ struct BlockStack {
     std::vector<HyRun> runs;
     std::vector<HyRot> rots;
     void *emb = nullptr, *head = nullptr;
-    float* fnorm = nullptr;  // final gain per channel
+    float *fnorm = nullptr, *fnorm_p = nullptr;  // final gain per channel; times sqrt(D / Dp)
     float fgain = 0.0f;
     std::map<std::string, bool> want;  // tensor -> placed
     bool dirty = true;
@@ -74,6 +78,9 @@ struct BlockStack {
     int32_t *nsegs = nullptr, *widx = nullptr;
     float *x = nullptr, *q = nullptr, *k = nullptr, *v = nullptr, *g = nullptr, *o = nullptr, *lg = nullptr;
     void *c1 = nullptr, *c2 = nullptr, *xl = nullptr;  // fp32 or fp16 by path
+    float* part = nullptr;   // split partials of the decode attention
+    float* bg_ws = nullptr;  // split-K partials and arrival counters of the batched projections
+    unsigned* bg_cnt = nullptr;
     std::vector<void*> allocs;
     std::vector<std::pair<hipGraph_t, hipGraphExec_t>> graphs_one, graphs_rows;
 };
@@ -121,10 +128,15 @@ static int hy_layer_init(HyLayer& l, int i) {
         l.e_v = l.e_k + d.heads * l.hpv;
         l.e_g = l.e_v + d.heads * l.hpv;
     }
-    l.u1p = pad_to(l.e_g, 64);  // 128 rows: a GEMM row block never straddles the two inputs
-    l.u2p = pad_to(d.ff, 64);
+    l.u1p = d.ff > 0 ? pad_to(l.e_g, kHySection) : pad_to(l.e_g, 8);
+    l.u2p = pad_to(d.ff, 8);
     return SLI_OK;
 }
+
+// decode attention splits per head at most (attn_mfma_tpw: at most kAmMaxSplits up to 64 tiles per wave)
+static int hy_attn_splits(int T) { return std::max(kAmMaxSplits, (T + 64 * kAmWgKeys - 1) / (64 * kAmWgKeys)); }
+
+static int hy_allow_lds();
 
 int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out) {
     const sli_stack_config& c = *cfg;
@@ -244,6 +256,7 @@ int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out)
     HY_TRY(hy_alloc(s, &s->emb, s->wb * (size_t)s->V * s->D));
     HY_TRY(hy_alloc(s, &s->head, s->wb * (size_t)s->Vp * s->Dp));
     HY_TRY(hy_alloc(s, (void**)&s->fnorm, sizeof(float) * s->Dp));
+    HY_TRY(hy_alloc(s, (void**)&s->fnorm_p, sizeof(float) * s->Dp));
     for (const char* n : {"embed", "head", "final.norm"}) s->want[n] = false;
     const size_t M = s->M;
     HY_TRY(hy_alloc(s, (void**)&s->rows, sizeof(RowRef) * M));
@@ -260,7 +273,26 @@ int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out)
     HY_TRY(hy_alloc(s, (void**)&s->g, sizeof(float) * M * nv));
     HY_TRY(hy_alloc(s, (void**)&s->o, sizeof(float) * M * no));
     HY_TRY(hy_alloc(s, (void**)&s->lg, sizeof(float) * M * s->V));
-    return SLI_OK;
+    const int Bp = s->B <= kBgMaxBatch ? s->B : pad_to(s->B, kHyTile);
+    size_t part = 0, bgp = 0, bgc = 1;
+    for (const HyLayer& l : s->layers) {
+        if (l.d.mixer == SLI_MIX_ATTENTION)
+            part = std::max(part, (size_t)Bp * l.d.heads * hy_attn_splits(s->T) * (l.hd + kAttnPartPad));
+        if (s->f16 && s->B > 1)
+            for (auto [np, K] : {std::make_pair(l.e_g, s->Dp), std::make_pair((int)l.d.ff, s->Dp),
+                                 std::make_pair((s->D + 1) / 2, l.Kp), std::make_pair((s->V + 1) / 2, s->Dp)})
+                for (int b = 2; b <= std::min(s->B, kBgMaxBatch); ++b) {
+                    if (np == 0) continue;
+                    const BgPlan p = bg_plan((np + 7) / 8, K, b, false, gemv_max_blocks());
+                    SLI_CHECK(p.groups > 0, SLI_ERR_SHAPE, "stack: no tiling of a batched projection fits");
+                    bgp = std::max(bgp, bg_part_bytes(p));
+                    bgc = std::max(bgc, (size_t)p.groups);
+                }
+    }
+    HY_TRY(hy_alloc(s, (void**)&s->part, sizeof(float) * part));
+    HY_TRY(hy_alloc(s, (void**)&s->bg_ws, bgp + 256));
+    HY_TRY(hy_alloc(s, (void**)&s->bg_cnt, sizeof(unsigned) * bgc));
+    return hy_allow_lds();
 }
 
 void hy_destroy(BlockStack* s) {
@@ -453,6 +485,8 @@ int hy_prepare(BlockStack* s) {
     std::vector<float> g(Dp, 0.0f);
     std::fill(g.begin(), g.begin() + s->D, s->fgain);
     SLI_HIP(hipMemcpy(s->fnorm, g.data(), sizeof(float) * Dp, hipMemcpyHostToDevice));
+    std::fill(g.begin(), g.begin() + s->D, (float)(s->fgain * std::sqrt((double)s->D / Dp)));
+    SLI_HIP(hipMemcpy(s->fnorm_p, g.data(), sizeof(float) * Dp, hipMemcpyHostToDevice));
     s->dirty = false;
     return SLI_OK;
 }
@@ -467,9 +501,74 @@ struct HyRec {
     int msegs;  // portions at most
     hipStream_t st() const { return s->stream; }
 
+    // How a projection over M rows runs: the batch-1 GEMV, the batched MFMA projection (2 .. 8 rows), the prompt GEMM
+    // (fp16, more rows), or the plain kernel (fp32, more than one row; widths past the GEMV's LDS stage).
+    enum Path { GV, BG, PG, RG };
+    static constexpr bool F16 = std::is_same<WT, __half>::value;
+    static Path path(int M, int K) {
+        if (M == 1 && K <= kGemvMaxCols) return GV;
+        if (!F16) return RG;
+        return M <= kBgMaxBatch ? (M == 1 ? RG : BG) : PG;
+    }
+    // rows of the launches for n rows
+    static int rows_for(int n) { return F16 && n > kBgMaxBatch ? pad_to(n, kHyTile) : n; }
+
     template <class Epi>
     int project(const void* W, const void* X, int K, int npairs, int u0, const Epi& e) const {
-        SLI_HIP((launch_rows_gemm<WT, Epi>((const WT*)W + (size_t)2 * u0 * K, (const float*)X, K, npairs, u0, M, e, st())));
+        const WT* w = (const WT*)W + (size_t)2 * u0 * K;
+        const Path p = path(M, K);
+        if (p == GV) {
+            GemvIn in{(const float*)X, nullptr, 0.0f, K};
+            SLI_HIP((launch_gemv_u<WT, 2, 4, true>(w, in, GvPair<Epi>{e, npairs, u0}, npairs, st())));
+            return SLI_OK;
+        }
+        if constexpr (F16) {
+            if (p == BG) {
+                BgIn in{};
+                in.x = (const float*)X;
+                in.K = K;
+                in.B = M;
+                in.ws = s->bg_ws;
+                in.counters = s->bg_cnt;
+                const BgPlan pl = bg_plan((npairs + 7) / 8, K, M, false, gemv_max_blocks());
+                SLI_HIP((launch_bgemm(w, in, BgPair<Epi>{e, npairs, u0}, pl, st())));
+                return SLI_OK;
+            }
+            if (p == PG) return pgemm(w, (const __half*)X, nullptr, 0, K, npairs, u0, e);
+        }
+        SLI_HIP((launch_rows_gemm<WT, Epi>(w, (const float*)X, K, npairs, u0, M, e, st())));
+        return SLI_OK;
+    }
+    // pairs [0, split) read X, pairs [split, npairs) X2 (split: a multiple of kHySection; X2 null: one input)
+    template <class Epi>
+    int pgemm(const WT* w, const __half* X, const __half* X2, int split, int K, int npairs, int u0, const Epi& e) const {
+        if constexpr (F16) {
+            PgIn<__half> in{w, X, nullptr, pad_to(2 * npairs, 16), K, M};
+            if (X2) in.Bhi2 = X2, in.row_b2 = 2 * split;
+            return pg_pick(M, [&](auto cfg) -> int {
+                SLI_HIP((launch_pgemm<PgPair<Epi>, decltype(cfg), __half>(in, PgPair<Epi>{e, npairs, u0}, nullptr, st())));
+                return SLI_OK;
+            });
+        } else {
+            return fail(SLI_ERR_ARG, "prompt GEMM: fp16 weights");
+        }
+    }
+    template <class F>
+    static int pg_pick(int M, F&& f) {
+        if (M % 128 == 0) return f(PgCfg<128, 2, 3, 4, true, 0, 1>{});
+        if (M % 64 == 0) return f(PgCfg<64, 2, 4, 2, true, 0, 1>{});
+        return f(PgCfg<32, 2, 4, 2, true, 0, 1>{});
+    }
+    template <class Epi>
+    static int allow() {
+        if constexpr (F16) {
+            for (int M : {32, 64, 128})
+                HY_TRY(pg_pick(M, [&](auto cfg) -> int {
+                    SLI_HIP((pgemm_allow_lds<PgPair<Epi>, decltype(cfg), __half>()));
+                    return SLI_OK;
+                }));
+            SLI_HIP((bg_allow_lds<BgPair<Epi>, false>()));
+        }
         return SLI_OK;
     }
     template <typename OT>
@@ -503,27 +602,109 @@ struct HyRec {
     template <typename OT>
     int mixer(const HyLayer& l, const HyRun& r) const {
         const sli_block_desc& d = l.d;
-        if (d.mixer == SLI_MIX_ATTENTION) {
-            AttnRowsArgs a{l.q, r.kc, r.vc, s->rows, l.r1, l.r2, l.sink, d.heads, d.kv_heads, d.dim, d.vdim, l.hd,
-                           s->T, M, d.scale};
-            hipLaunchKernelGGL((attn_rows_kernel<KT, OT>), dim3(d.heads, M), dim3(64), sizeof(float) * (d.dim + 64), st(),
-                               a, cat<OT>(l), l.Kp);
-        } else {
-            RetArgs a{s->q, s->k, s->v, r.S, s->o, l.decay, s->rows, s->segs, s->nsegs, d.heads, d.dim, d.vdim, l.nsl};
-            if (one)
-                hipLaunchKernelGGL(ret_step_kernel, dim3(l.nsl, d.heads, M), dim3(256), 0, st(), a);
-            else
-                hipLaunchKernelGGL(ret_scan_kernel, dim3(l.nsl, d.heads, msegs), dim3(256), ret_scan_lds(d.dim), st(), a);
-            SLI_HIP(hipGetLastError());
-            hipLaunchKernelGGL(ret_gate_kernel<OT>, dim3((M * d.heads + 3) / 4), dim3(256), 0, st(), s->o, s->g, s->rows,
-                               cat<OT>(l), l.Kp, M, d.heads, d.vdim, s->c.eps);
+        if (d.mixer == SLI_MIX_ATTENTION) return attention<OT>(l, r);
+        RetArgs a{s->q, s->k, s->v, r.S, s->o, l.decay, s->rows, s->segs, s->nsegs, d.heads, d.dim, d.vdim, l.nsl};
+        const dim3 sg(l.nsl, d.heads, msegs);
+        const int kd = F16 ? ret_chunk_kd(d.dim) : 0;
+        if (one)
+            hipLaunchKernelGGL(ret_step_kernel, dim3(l.nsl, d.heads, M), dim3(256), 0, st(), a);
+        else if (kd == 32)
+            hipLaunchKernelGGL(ret_chunk_kernel<32>, sg, dim3(256), RcGeo<32>::LDS, st(), a);
+        else if (kd == 64)
+            hipLaunchKernelGGL(ret_chunk_kernel<64>, sg, dim3(256), RcGeo<64>::LDS, st(), a);
+        else if (kd == 128)
+            hipLaunchKernelGGL(ret_chunk_kernel<128>, sg, dim3(256), RcGeo<128>::LDS, st(), a);
+        else if (kd == 256)
+            hipLaunchKernelGGL(ret_chunk_kernel<256>, sg, dim3(256), RcGeo<256>::LDS, st(), a);
+        else
+            hipLaunchKernelGGL(ret_scan_kernel, sg, dim3(256), ret_scan_lds(d.dim), st(), a);
+        SLI_HIP(hipGetLastError());
+        hipLaunchKernelGGL(ret_gate_kernel<OT>, dim3((M * d.heads + 3) / 4), dim3(256), 0, st(), s->o, s->g, s->rows,
+                           cat<OT>(l), l.Kp, M, d.heads, d.vdim, s->c.eps);
+        SLI_HIP(hipGetLastError());
+        return SLI_OK;
+    }
+    template <int HD>
+    void attn_split(const AttnArgs<__half>& a, int g, int blocks, bool ring) const {
+        const dim3 gr(blocks), bl(64 * kAmWaves);
+        switch (g * 2 + (ring ? 1 : 0)) {
+            case 2: hipLaunchKernelGGL((attn_mfma_kernel<HD, 1, 1, true>), gr, bl, 0, st(), a); break;
+            case 3: hipLaunchKernelGGL((attn_mfma_kernel<HD, 1, 2, true>), gr, bl, 0, st(), a); break;
+            case 4: hipLaunchKernelGGL((attn_mfma_kernel<HD, 2, 1, true>), gr, bl, 0, st(), a); break;
+            case 5: hipLaunchKernelGGL((attn_mfma_kernel<HD, 2, 2, true>), gr, bl, 0, st(), a); break;
+            case 8: hipLaunchKernelGGL((attn_mfma_kernel<HD, 4, 1, true>), gr, bl, 0, st(), a); break;
+            case 9: hipLaunchKernelGGL((attn_mfma_kernel<HD, 4, 2, true>), gr, bl, 0, st(), a); break;
+            case 16: hipLaunchKernelGGL((attn_mfma_kernel<HD, 8, 1, true>), gr, bl, 0, st(), a); break;
+            default: hipLaunchKernelGGL((attn_mfma_kernel<HD, 8, 2, true>), gr, bl, 0, st(), a); break;
         }
+    }
+    template <typename OT>
+    int attention(const HyLayer& l, const HyRun& r) const {
+        const sli_block_desc& d = l.d;
+        const AttnRowsArgs ra{l.q, r.kc, r.vc, s->rows, l.r1, l.r2, l.sink, d.heads, d.kv_heads, d.dim, d.vdim, l.hd,
+                              s->T, M, d.scale};
+        if constexpr (F16) {
+            if (one && l.hd <= 128) {  // split context, then the merge with the sink
+                const int gq = d.heads / d.kv_heads, g = gq % 8 == 0 ? 8 : gq % 4 == 0 ? 4 : gq % 2 == 0 ? 2 : 1;
+                const int kvg = gq / g, nkv = M * d.kv_heads * kvg;
+                AttnArgs<__half> a{};
+                a.q = l.q;
+                a.k = (const __half*)r.kc;
+                a.v = (const __half*)r.vc;
+                a.pos_stride = l.hd;
+                a.head_stride = (long long)s->T * l.hd;
+                a.part = s->part;
+                a.pos_dev = &s->rows->pos;
+                a.slot_dev = &s->rows->slot;
+                a.pos_seq_stride = sizeof(RowRef) / sizeof(int32_t);
+                a.n_kv_heads = nkv;
+                a.seq_heads = d.kv_heads * kvg;
+                a.kv_group = kvg;
+                a.scale = d.scale;
+                a.bias_r1 = l.r1;
+                a.bias_r2 = l.r2;
+                const int tpw = attn_mfma_tpw(nkv, s->T, device_cus());
+                a.ppwg = kAmWgKeys * tpw;
+                a.max_splits = (s->T + a.ppwg - 1) / a.ppwg;
+                SLI_CHECK(a.max_splits <= hy_attn_splits(s->T), SLI_ERR_SHAPE, "attention: more splits than the buffer holds");
+                if (l.hd == 64)
+                    attn_split<64>(a, g, nkv * a.max_splits, tpw > 1);
+                else
+                    attn_split<128>(a, g, nkv * a.max_splits, tpw > 1);
+                SLI_HIP(hipGetLastError());
+                hipLaunchKernelGGL(attn_sink_merge_kernel<OT>, dim3(d.heads, M), dim3(128), 0, st(), s->part, ra,
+                                   a.max_splits, a.ppwg, cat<OT>(l), l.Kp);
+                SLI_HIP(hipGetLastError());
+                return SLI_OK;
+            }
+            if constexpr (!std::is_same<OT, float>::value) {
+                if (!one && l.hd <= 128) {
+                    const PfAttnArgs<__half> pa{l.q, (const __half*)r.kc, (const __half*)r.vc, cat<OT>(l), nullptr,
+                                                d.heads, d.kv_heads, s->T, d.scale};
+                    const PfRowsArgs px{s->rows, l.r1, l.r2, l.sink, l.Kp, d.vdim};
+                    const dim3 gr(M / 16, d.heads);
+                    if (l.hd == 64)
+                        hipLaunchKernelGGL((pf_attn_mfma_kernel<64, true>), gr, dim3(256), 0, st(), pa, nullptr, px);
+                    else
+                        hipLaunchKernelGGL((pf_attn_mfma_kernel<128, true>), gr, dim3(256), 0, st(), pa, nullptr, px);
+                    SLI_HIP(hipGetLastError());
+                    return SLI_OK;
+                }
+            }
+        }
+        hipLaunchKernelGGL((attn_rows_kernel<KT, OT>), dim3(d.heads, M), dim3(64), sizeof(float) * (d.dim + 64), st(), ra,
+                           cat<OT>(l), l.Kp);
         SLI_HIP(hipGetLastError());
         return SLI_OK;
     }
     int layer(const HyRun& r) const {
+        if constexpr (F16)
+            if (M > kBgMaxBatch) return layer_as<__half>(r);
+        return layer_as<float>(r);
+    }
+    template <typename OT>
+    int layer_as(const HyRun& r) const {
         const HyLayer& l = s->layers[r.layer];
-        using OT = float;
         const CanonArgs ca = canon(l, r);
         hipLaunchKernelGGL(canon_rows_kernel<OT>, dim3(M), dim3(256), 0, st(), ca, (OT*)s->c1,
                            l.d.ff > 0 ? (OT*)s->c2 : (OT*)nullptr, one ? 1 : 0);
@@ -533,9 +714,24 @@ struct HyRec {
             SLI_HIP(hipGetLastError());
         }
         const auto ei = in_epi<OT>(l, r);
-        HY_TRY(project(l.win, s->c1, s->Dp, l.e_g, 0, ei));
-        if (l.d.ff > 0) HY_TRY(project(l.win, s->c2, s->Dp, l.d.ff, l.u1p, ei));
+        if constexpr (!std::is_same<OT, float>::value) {
+            if (l.d.ff > 0)
+                HY_TRY(pgemm((const WT*)l.win, (const __half*)s->c1, (const __half*)s->c2, l.u1p, s->Dp, l.u1p + l.d.ff, 0, ei));
+            else
+                HY_TRY(pgemm((const WT*)l.win, (const __half*)s->c1, nullptr, 0, s->Dp, l.e_g, 0, ei));
+        } else {
+            HY_TRY(project(l.win, s->c1, s->Dp, l.e_g, 0, ei));
+            if (l.d.ff > 0) HY_TRY(project(l.win, s->c2, s->Dp, l.d.ff, l.u1p, ei));
+        }
         HY_TRY(mixer<OT>(l, r));
+        if constexpr (std::is_same<OT, float>::value) {
+            if (path(M, l.Kp) == GV) {
+                GemvIn in{l.cat32, nullptr, 0.0f, l.Kp};
+                const EpiStore<1> e{s->x, s->x, nullptr, s->c.residual_mult, s->D};
+                SLI_HIP((launch_gemv_u<WT, 1, 6, true>((const WT*)l.wout, in, e, s->D, st())));
+                return SLI_OK;
+            }
+        }
         const HyOut eo{s->x, s->Dp, s->D, s->c.residual_mult};
         return project(l.wout, cat<OT>(l), l.Kp, (s->D + 1) / 2, 0, eo);
     }
@@ -547,30 +743,56 @@ struct HyRec {
     }
     // logits [n][V] of rows idx (null: rows 0 .. n - 1)
     int logits(const int32_t* idx, int n, float* y) const {
-        using OT = float;
+        HyRec h = *this;
+        h.M = rows_for(n);
+        if constexpr (F16)
+            if (h.M > kBgMaxBatch) return h.template logits_as<__half>(idx, n, y);
+        return h.template logits_as<float>(idx, n, y);
+    }
+    template <typename OT>
+    int logits_as(const int32_t* idx, int n, float* y) const {
         hipLaunchKernelGGL(norm_rows_kernel<OT>, dim3(n), dim3(256), 0, st(), s->x, idx, s->fnorm, (OT*)s->xl, s->D, s->Dp,
                            s->c.eps);
         SLI_HIP(hipGetLastError());
-        HyRec h = *this;
-        h.M = n;
-        return h.project(s->head, s->xl, s->Dp, (s->V + 1) / 2, 0, HyLogits{y, s->V, n});
+        return project(s->head, s->xl, s->Dp, (s->V + 1) / 2, 0, HyLogits{y, s->V, n});
     }
     int pass() const {
         HY_TRY(embed());
         for (const HyRun& r : s->runs) HY_TRY(layer(r));
         return SLI_OK;
     }
-    int step(const DevState* dst, float* y, unsigned long long* keys, int key_ld, int* nkeys) const {
-        hipLaunchKernelGGL(hy_rows_kernel, dim3(1), dim3(64), 0, st(), dst, s->rows, M);
+    int step(const DevState* dst, int B, float* y, unsigned long long* keys, int key_ld, int* nkeys) const {
+        hipLaunchKernelGGL(hy_rows_kernel, dim3(1), dim3(64), 0, st(), dst, s->rows, B, M);
         SLI_HIP(hipGetLastError());
         HY_TRY(pass());
-        HY_TRY(logits(nullptr, M, y));
-        hipLaunchKernelGGL(hy_keys_kernel, dim3(M), dim3(256), 0, st(), y, s->V, keys, key_ld);
+        if (B == 1 && path(1, s->Dp) == GV) {
+            // the norm over the padded row: x / sqrt(sum / D + eps) = sqrt(D / Dp) x / sqrt(sum / Dp + eps D / Dp)
+            GemvIn in{s->x, s->fnorm_p, (float)((double)s->c.eps * s->D / s->Dp), s->Dp};
+            const EpiLogits<2> e{y, keys, nullptr, s->V, 0, 0ull};
+            const int units = (s->V + 1) / 2, cs = gemv_split<WT, 4>(units, s->Dp).cs;
+            *nkeys = cs == 1 ? gemv_balanced_blocks(units) : gemv_blocks(units, cs);  // launch_gemv's grid
+            SLI_HIP((launch_gemv_u<WT, 2, 4, true>((const WT*)s->head, in, e, units, st())));
+            return SLI_OK;
+        }
+        HY_TRY(logits(nullptr, B, y));
+        hipLaunchKernelGGL(hy_keys_kernel, dim3(B), dim3(256), 0, st(), y, s->V, keys, key_ld);
         SLI_HIP(hipGetLastError());
         *nkeys = 1;
         return SLI_OK;
     }
+    static int allow_all() {
+        HY_TRY((allow<HyIn<KT, float>>()));
+        HY_TRY((allow<HyIn<KT, __half>>()));
+        HY_TRY((allow<HyOut>()));
+        return allow<HyLogits>();
+    }
 };
+
+static int hy_allow_lds() {
+    SLI_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&ret_chunk_kernel<256>),
+                                hipFuncAttributeMaxDynamicSharedMemorySize, (int)RcGeo<256>::LDS));
+    return HyRec<__half>::allow_all();
+}
 
 #define HY_DISPATCH(s, M, one, msegs, CALL) \
     ((s)->f16 ? HyRec<__half>{(s), (M), (one), (msegs)}.CALL : HyRec<float>{(s), (M), (one), (msegs)}.CALL)
@@ -579,7 +801,8 @@ int hy_key_ld(const BlockStack*, int) { return std::max(1, gemv_max_blocks()); }
 
 int hy_record_step(BlockStack* s, const DevState* st, int B, float* logits, unsigned long long* keys, int key_ld,
                    int* nkeys) {
-    return HY_DISPATCH(s, B, true, B, step(st, logits, keys, key_ld, nkeys));
+    const int M = s->f16 ? HyRec<__half>::rows_for(B) : B;
+    return HY_DISPATCH(s, M, true, M, step(st, B, logits, keys, key_ld, nkeys));
 }
 
 static int hy_capture(BlockStack* s, std::pair<hipGraph_t, hipGraphExec_t>& g, int M, bool one, int msegs) {
@@ -602,7 +825,8 @@ int hy_pass(BlockStack* s, const std::vector<RowRef>& rows_in, const std::vector
     const int n = (int)rows_in.size();
     SLI_CHECK(n >= 1 && n <= s->M && !segs.empty() && (int)segs.size() <= s->M, SLI_ERR_SHAPE, "pass: too many rows");
     // a decode step runs its rows as they are; a prompt pass is padded to a row count with a captured graph
-    int M = n, gi = n - 1;
+    int M = s->f16 ? HyRec<__half>::rows_for(n) : n, gi = M - 1;
+    SLI_CHECK(!one || n <= s->B, SLI_ERR_SHAPE, "pass: more sequences than slots");
     if (!one) {
         M = kHyTile, gi = 0;
         while (M < n) M *= 2, ++gi;

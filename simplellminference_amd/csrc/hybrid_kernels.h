@@ -17,9 +17,13 @@ namespace sli {
 
 // ---------------------------------------------------------------- embedding
 // rows of a decode step from the engine's states: one row per slot
-__global__ void hy_rows_kernel(const DevState* st, RowRef* rows, int B) {
+// (rows B .. M - 1: padding)
+__global__ void hy_rows_kernel(const DevState* st, RowRef* rows, int B, int M) {
     const int b = threadIdx.x;
-    if (b < B) rows[b] = RowRef{b, st[b].pos, st[b].token, b};
+    if (b < B)
+        rows[b] = RowRef{b, st[b].pos, st[b].token, b};
+    else if (b < M)
+        rows[b] = RowRef{-1, 0, 0, b};
 }
 
 template <typename WT>

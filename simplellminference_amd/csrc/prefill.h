@@ -27,6 +27,7 @@
 // chunk size serves every chunk of every prompt.
 #pragma once
 #include "common.h"
+#include "step_state.h"
 
 namespace sli {
 
@@ -135,6 +136,9 @@ struct PgIn {
     const __half* Bhi;  // [M][K] activations, fp16 hi
     const __half* Blo;  // [M][K] fp16 lo
     int N, K, M;        // rows, depth, chunk rows (a multiple of BM)
+    // weight rows from row_b2 on (a multiple of the tiling's BN) read their activations from Bhi2 (one image only)
+    const __half* Bhi2 = nullptr;
+    int row_b2 = 0x7fffffff;
 };
 
 // Tiling: a workgroup of 2 WR waves owns BN = 32 WR weight rows x BM chunk rows; wave w holds the 2 x BM/32
@@ -153,15 +157,17 @@ struct PgIn {
 // SA_ > 0 (PIPE only): the weight (A) images get a ring of their own, SA_ stages deep (SA_ - 1 issued ahead), and
 // the activation (B) images a 2-stage ring (one ahead): the A bytes come from HBM (read once per chunk), the B bytes
 // from L2, so only A needs the deep prefetch, and B, the larger image, does not pay for it in LDS.
-template <int BM_, int WR_, int S_, int AT_ = 2, bool PIPE_ = false, int SA_ = 0>
+// NB_: activation images per position: 2 (fp16 hi + lo, two MFMAs per product) or 1 (fp16 activations; PIPE only).
+template <int BM_, int WR_, int S_, int AT_ = 2, bool PIPE_ = false, int SA_ = 0, int NB_ = 2>
 struct PgCfg {
-    static constexpr int BM = BM_, WR = WR_, S = S_, AT = AT_, SA = SA_;
+    static_assert(NB_ == 2 || (NB_ == 1 && PIPE_), "activation images");
+    static constexpr int BM = BM_, WR = WR_, S = S_, AT = AT_, SA = SA_, NB = NB_;
     static constexpr bool PIPE = PIPE_;
 };
 
 template <class Cfg, typename WT>
 struct PgGeo {
-    static constexpr int BM = Cfg::BM, WR = Cfg::WR, S = Cfg::S, AT = Cfg::AT;
+    static constexpr int BM = Cfg::BM, WR = Cfg::WR, S = Cfg::S, AT = Cfg::AT, NB = Cfg::NB;
     static constexpr int WAVES = 2 * WR, THREADS = 64 * WAVES, BN = 16 * AT * WR;
     static constexpr int KS = sizeof(WT) == 1 ? 128 : 64;  // depth per stage
     static constexpr int KBS = KS / 32;                    // MFMA k-blocks per stage
@@ -172,7 +178,7 @@ struct PgGeo {
     static constexpr int WPT = PT / 2;  // per wave
     static constexpr int NA = AT * WR;  // weight row tiles
     static constexpr int A_BYTES = NA * A_IMG;
-    static constexpr int STAGE = A_BYTES + 2 * PT * B_IMG;
+    static constexpr int STAGE = A_BYTES + NB * PT * B_IMG;
     static constexpr int NDMA = STAGE / 1024;  // wave-instructions per stage
     static constexpr int DPW = NDMA / WAVES;   // per wave
     static constexpr int SA = Cfg::SA;         // split rings (PgCfg): A pieces per wave DPA, B pieces DPB
@@ -269,10 +275,10 @@ __global__ void __launch_bounds__(128 * Cfg::WR) pgemm_kernel(PgIn<WT> in, Epi e
         } else {
             constexpr int cpr = Geo::B_ROW / 16;
             const int o2 = off - Geo::A_BYTES;
-            const int u = o2 / Geo::B_IMG, pt = u >> 1;
+            const int u = o2 / Geo::B_IMG, pt = Geo::NB == 2 ? u >> 1 : u;
             const int r = (o2 % Geo::B_IMG) / Geo::B_ROW + lane / cpr;
             const int c = (lane % cpr) ^ pg_swz(r, Geo::B_ROW);
-            const __half* B = (u & 1) ? in.Blo : in.Bhi;
+            const __half* B = Geo::NB == 2 ? ((u & 1) ? in.Blo : in.Bhi) : rb * Geo::BN >= in.row_b2 ? in.Bhi2 : in.Bhi;
             const int m = pb * BM + pt * 16 + r;
             src[j] = reinterpret_cast<const char*>(B) + (size_t)m * in.K * 2 + c * 16;
             adv[j] = Geo::B_ROW;
@@ -343,9 +349,9 @@ __global__ void __launch_bounds__(128 * Cfg::WR) pgemm_kernel(PgIn<WT> in, Epi e
 #pragma unroll
         for (int b = 0; b < Geo::WPT; ++b) {
             const int pt = wp * Geo::WPT + b;
-            const char* img = stb + (2 * pt) * Geo::B_IMG + r16 * Geo::B_ROW + ((4 * kb + kg) ^ sb) * 16;
+            const char* img = stb + (Geo::NB * pt) * Geo::B_IMG + r16 * Geo::B_ROW + ((4 * kb + kg) ^ sb) * 16;
             bh[b] = *reinterpret_cast<const u32x4*>(img);
-            bl[b] = *reinterpret_cast<const u32x4*>(img + Geo::B_IMG);
+            if constexpr (Geo::NB == 2) bl[b] = *reinterpret_cast<const u32x4*>(img + Geo::B_IMG);
         }
     };
     auto mfmas = [&](const u32x4(&af)[AT], const u32x4(&bh)[Geo::WPT], const u32x4(&bl)[Geo::WPT]) {
@@ -353,10 +359,12 @@ __global__ void __launch_bounds__(128 * Cfg::WR) pgemm_kernel(PgIn<WT> in, Epi e
         for (int b = 0; b < Geo::WPT; ++b)
 #pragma unroll
             for (int a = 0; a < AT; ++a) acc[a][b] = pf_mfma(af[a], bh[b], acc[a][b]);
+        if constexpr (Geo::NB == 2) {
 #pragma unroll
-        for (int b = 0; b < Geo::WPT; ++b)
+            for (int b = 0; b < Geo::WPT; ++b)
 #pragma unroll
-            for (int a = 0; a < AT; ++a) acc[a][b] = pf_mfma(af[a], bl[b], acc[a][b]);
+                for (int a = 0; a < AT; ++a) acc[a][b] = pf_mfma(af[a], bl[b], acc[a][b]);
+        }
     };
     if constexpr (Cfg::PIPE) {
         // set X holds even k-blocks, set Y odd ones (KBS is even; an int8 half stage has KBS / 2 = 2): per stage
@@ -700,8 +708,18 @@ __device__ __forceinline__ uint2 pa_tr_read(unsigned lds_addr) {
     return v;
 }
 
-template <int HD>
-__global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a, const PfState* __restrict__ ps) {
+//
+// ROWS: the rows are packed portions of several sequences (step_state.h RowRef; a 16-row group belongs to one portion,
+// its valid rows first), with a distance bias and a sink per head (attn_rows.h) and one fp16 output [M][ldo] of vdim
+// dims per head; the caches hold one [hkv][T][HD] block per sequence slot.
+struct PfRowsArgs {
+    const RowRef* rows = nullptr;
+    const float *r1 = nullptr, *r2 = nullptr, *sink = nullptr;  // [hq]
+    int ldo = 0, vdim = 0;
+};
+template <int HD, bool ROWS = false>
+__global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a, const PfState* __restrict__ ps,
+                                                           PfRowsArgs x) {
     using G = PaGeo<HD>;
     constexpr int ND = HD / 32, NT = HD / 16;  // 32-d blocks (S), 16-d tiles (O)
     __shared__ __attribute__((aligned(1024))) char sm[4 * G::WAVE];
@@ -709,10 +727,26 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
     const int wave = __builtin_amdgcn_readfirstlane((int)(threadIdx.x >> 6));
     const int g = lane >> 4, i16 = lane & 15;
     const int h = blockIdx.y, kvh = h / (a.hq / a.hkv);
-    const int p0 = ps->p0;
     const int mq = blockIdx.x * 16 + i16;  // this lane's query (chunk row)
-    const int pos = p0 + mq;
-    const int last = min(p0 + blockIdx.x * 16 + 15, a.T - 1);  // the group's last query position
+    int pos, last, slot = 0;  // last: the group's last query position
+    bool live = true;
+    if constexpr (ROWS) {
+        const RowRef r0 = x.rows[blockIdx.x * 16];
+        if (r0.slot < 0) return;  // (uniform) a group of padding rows
+        slot = r0.slot;
+        live = x.rows[mq].slot >= 0;
+        pos = r0.pos + i16;
+        last = r0.pos + (int)__popcll(__ballot(live)) / 4 - 1;  // (a row is the query of 4 lanes)
+    } else {
+        pos = ps->p0 + mq;
+        last = min(ps->p0 + (int)blockIdx.x * 16 + 15, a.T - 1);
+    }
+    const int kmax = ROWS ? last : a.T - 1;  // cache rows past it are read as this one (their scores are masked)
+    float bias1 = 0.0f, bias2 = 0.0f;
+    if constexpr (ROWS) {
+        bias1 = x.r1[h];
+        bias2 = x.r2[h];
+    }
     const int ntiles = last / 32 + 1;
     const size_t qs = (size_t)a.hq * HD;
     // Qᵀ as the B operand: lane l = query l & 15, d = 32 db + 8 g .. +8, fp32 -> hi + lo
@@ -735,8 +769,8 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
     char* kimg = sm + wave * G::WAVE;
     const unsigned kbase = (unsigned)(uintptr_t)(const __attribute__((address_space(3))) char*)kimg;
     const unsigned vbase = kbase + G::IMG;
-    const __half* kc = a.kc + (size_t)kvh * a.T * HD;
-    const __half* vc = a.vc + (size_t)kvh * a.T * HD;
+    const __half* kc = a.kc + ((size_t)slot * a.hkv + kvh) * a.T * HD;
+    const __half* vc = a.vc + ((size_t)slot * a.hkv + kvh) * a.T * HD;
     for (int tt = wave; tt < ntiles; tt += 4) {
         const int t0 = tt * 32;
         // K pieces 0 .. P/2-1, V pieces P/2 .. P-1; lane i of a piece: row (piece rows) + i / CPR, physical
@@ -747,7 +781,7 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
             const int jj = isv ? j - G::PIECES / 2 : j;
             const int r = jj * (1024 / G::ROWB) + lane / G::CPR;
             const int c = (lane % G::CPR) ^ (isv ? pa_swz_v(r, G::ROWB) : pa_swz_k(r, G::ROWB));
-            const __half* src = (isv ? vc : kc) + (size_t)min(t0 + r, a.T - 1) * HD + c * 8;
+            const __half* src = (isv ? vc : kc) + (size_t)min(t0 + r, kmax) * HD + c * 8;
             pf_dma(src, (isv ? vbase : kbase) + (unsigned)(jj * 1024));
         }
         pf_wait_vm<0>();
@@ -773,7 +807,9 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int key = t0 + kt * 16 + 4 * g + r;
-                const float v = key <= pos ? sacc[kt][r] * a.scale : -INFINITY;
+                float sc = sacc[kt][r] * a.scale;
+                if constexpr (ROWS) sc -= bias1 * __logf(1.0f + bias2 * (float)(pos - key));
+                const float v = key <= pos ? sc : -INFINITY;
                 sv[kt * 4 + r] = v;
                 cmax = fmaxf(cmax, v);
             }
@@ -835,6 +871,10 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
         M = fmaxf(M, m4[w]);
     }
     float L = 0.0f;
+    if constexpr (ROWS) {
+        M = fmaxf(M, x.sink[h]);
+        L = expf(x.sink[h] - M);
+    }
 #pragma unroll
     for (int w = 0; w < 4; ++w) {
         w4[w] = m4[w] == -INFINITY ? 0.0f : expf(m4[w] - M);
@@ -846,6 +886,21 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
 #pragma unroll
         for (int w = 0; w < 4; ++w) acc += *reinterpret_cast<const pf_float4*>(fo + ((w * NT + t) * 64 + lane) * 4) * w4[w];
         // lane holds d = 16 t + 4 g + r of query mq
+        if constexpr (ROWS) {
+            const int d0 = t * 16 + 4 * g;
+            __half* dst = a.ohi + (size_t)mq * x.ldo + (size_t)h * x.vdim + d0;
+            if (!live) continue;
+            if (x.vdim % 4 == 0 && d0 < x.vdim) {
+                const __half hv[4] = {__float2half_rn(acc[0] * inv), __float2half_rn(acc[1] * inv),
+                                      __float2half_rn(acc[2] * inv), __float2half_rn(acc[3] * inv)};
+                *reinterpret_cast<uint2*>(dst) = *reinterpret_cast<const uint2*>(hv);
+            } else {
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    if (d0 + r < x.vdim) dst[r] = __float2half_rn(acc[r] * inv);
+            }
+            continue;
+        }
         const size_t idx = (size_t)mq * qs + (size_t)h * HD + t * 16 + 4 * g;
         __half hh[4], hl[4];
 #pragma unroll
