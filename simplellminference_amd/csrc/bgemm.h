@@ -140,6 +140,12 @@ __device__ __forceinline__ float bg_load_sc1(const float* base, unsigned bytes, 
     return __builtin_bit_cast(float, __builtin_amdgcn_raw_buffer_load_b32(rsrc, off, 0, 16 /* sc1 */));
 }
 
+// The fp32-rounded product (rms_kernel.cpp:20-22 stores it): not fused into the fp16 conversions that follow it
+__device__ __forceinline__ float bg_mul_rn(float a, float b) {
+#pragma clang fp contract(off)
+    return a * b;
+}
+
 // fp32 -> (fp16 hi, fp16 lo), hi + lo == v to ~2^-22 relative
 __device__ __forceinline__ void bg_split8(const float* y, u32x4& hi, u32x4& lo) {
     unsigned h[4], l[4];
@@ -279,7 +285,7 @@ __global__ void __launch_bounds__(kBgThreads) bgemm_kernel(const __half* __restr
             const float wv[8] = {wn[n][0].x, wn[n][0].y, wn[n][0].z, wn[n][0].w,
                                  wn[n][1].x, wn[n][1].y, wn[n][1].z, wn[n][1].w};
 #pragma unroll
-            for (int e = 0; e < 8; ++e) y[e] = y[e] * wv[e];
+            for (int e = 0; e < 8; ++e) y[e] = bg_mul_rn(y[e], wv[e]);
         }
         if (seq_live && bw < wnb) {
             u32x4 hi, lo;

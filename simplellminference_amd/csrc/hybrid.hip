@@ -309,23 +309,34 @@ void hy_destroy(BlockStack* s) {
 int hy_runs(const BlockStack* s) { return (int)s->runs.size(); }
 
 // ---------------------------------------------------------------- weights
+// where a tensor's elements come from: host memory, or (host null) a generator on the device
+struct HyFill {
+    const float* host = nullptr;
+    HySrcRand rand{};
+};
+
 static int hy_place(BlockStack* s, void* dst, int ld, int col0, const std::vector<int32_t>& map, int ncols,
-                    const float* host) {
+                    const HyFill& f) {
     const size_t n = map.size() * (size_t)ncols;
     float* tmp = nullptr;
     int32_t* dm = nullptr;
     int rc = SLI_OK;
-    if (hipMalloc(&tmp, sizeof(float) * n) != hipSuccess || hipMalloc(&dm, sizeof(int32_t) * map.size()) != hipSuccess)
+    if ((f.host && hipMalloc(&tmp, sizeof(float) * n) != hipSuccess) ||
+        hipMalloc(&dm, sizeof(int32_t) * map.size()) != hipSuccess)
         rc = fail(SLI_ERR_NOMEM, "weight staging");
-    if (rc == SLI_OK && (hipMemcpy(tmp, host, sizeof(float) * n, hipMemcpyHostToDevice) != hipSuccess ||
+    if (rc == SLI_OK && ((f.host && hipMemcpy(tmp, f.host, sizeof(float) * n, hipMemcpyHostToDevice) != hipSuccess) ||
                          hipMemcpy(dm, map.data(), sizeof(int32_t) * map.size(), hipMemcpyHostToDevice) != hipSuccess))
         rc = fail(SLI_ERR_HIP, "weight upload");
     if (rc == SLI_OK) {
-        const dim3 grid((unsigned)map.size());
+        const dim3 grid((unsigned)map.size()), bl(256);
+        auto go = [&](auto* d, auto src) {
+            using WT = std::remove_pointer_t<decltype(d)>;
+            hipLaunchKernelGGL((hy_place_kernel<WT, decltype(src)>), grid, bl, 0, s->stream, d, ld, col0, dm, ncols, src);
+        };
         if (s->f16)
-            hipLaunchKernelGGL(hy_place_kernel<__half>, grid, dim3(256), 0, s->stream, (__half*)dst, ld, col0, dm, ncols, tmp);
+            f.host ? go((__half*)dst, HySrcBuf{tmp}) : go((__half*)dst, f.rand);
         else
-            hipLaunchKernelGGL(hy_place_kernel<float>, grid, dim3(256), 0, s->stream, (float*)dst, ld, col0, dm, ncols, tmp);
+            f.host ? go((float*)dst, HySrcBuf{tmp}) : go((float*)dst, f.rand);
         if (hipGetLastError() != hipSuccess || hipStreamSynchronize(s->stream) != hipSuccess)
             rc = fail(SLI_ERR_HIP, "weight placement");
     }
@@ -384,7 +395,8 @@ static void hy_shape(const BlockStack* s, const std::string& name, int* li, std:
     else if (t == "mlp.down") set(s->D, d.ff);
 }
 
-int hy_set_tensor(BlockStack* s, const std::string& name, const float* host, int64_t n) {
+static int hy_put(BlockStack* s, const std::string& name, const HyFill& f, int64_t n) {
+    const float* host = f.host;  // (vectors always come from the host)
     auto it = s->want.find(name);
     SLI_CHECK(it != s->want.end(), SLI_ERR_ARG, "the model has no tensor '" + name + "'");
     int li;
@@ -392,15 +404,15 @@ int hy_set_tensor(BlockStack* s, const std::string& name, const float* host, int
     int64_t rows, cols;
     hy_shape(s, name, &li, &t, &rows, &cols);
     SLI_CHECK(n == rows * cols, SLI_ERR_SHAPE, "tensor '" + name + "' has the wrong size");
-    if (s->f16)
+    if (s->f16 && host)
         for (int64_t i = 0; i < n; ++i)
             SLI_CHECK(std::fabs(host[i]) <= 65504.0f, SLI_ERR_RANGE, "tensor '" + name + "' has values fp16 cannot hold");
     s->dirty = true;
     int rc = SLI_OK;
     if (name == "embed") {
-        rc = hy_place(s, s->emb, s->D, 0, strided_rows(s->V, 0, 1), s->D, host);
+        rc = hy_place(s, s->emb, s->D, 0, strided_rows(s->V, 0, 1), s->D, f);
     } else if (name == "head") {
-        rc = hy_place(s, s->head, s->Dp, 0, strided_rows(s->V, 0, 1), s->D, host);
+        rc = hy_place(s, s->head, s->Dp, 0, strided_rows(s->V, 0, 1), s->D, f);
     } else if (name == "final.norm") {
         s->fgain = host[0];
     } else {
@@ -412,14 +424,14 @@ int hy_set_tensor(BlockStack* s, const std::string& name, const float* host, int
         else if (t == "norm2") l.n2 = host[0];
         else if (t == "canon1") l.c1.assign(host, host + n);
         else if (t == "canon2") l.c2.assign(host, host + n);
-        else if (t == "mix.q") rc = hy_place(s, l.win, s->Dp, 0, head_rows(d.heads, d.dim, rh, 0), s->D, host);
-        else if (t == "mix.k") rc = hy_place(s, l.win, s->Dp, 0, head_rows(kvh, d.dim, rh, l.e_q), s->D, host);
-        else if (t == "mix.v") rc = hy_place(s, l.win, s->Dp, 0, head_rows(kvh, d.vdim, 0, l.e_k), s->D, host);
-        else if (t == "mix.g") rc = hy_place(s, l.win, s->Dp, 0, head_rows(d.heads, d.vdim, 0, l.e_v), s->D, host);
-        else if (t == "mix.o") rc = hy_place(s, l.wout, l.Kp, 0, strided_rows(s->D, 0, 1), l.mixw, host);
-        else if (t == "mlp.gate") rc = hy_place(s, l.win, s->Dp, 0, strided_rows(d.ff, 2 * l.u1p, 2), s->D, host);
-        else if (t == "mlp.up") rc = hy_place(s, l.win, s->Dp, 0, strided_rows(d.ff, 2 * l.u1p + 1, 2), s->D, host);
-        else if (t == "mlp.down") rc = hy_place(s, l.wout, l.Kp, l.KA, strided_rows(s->D, 0, 1), d.ff, host);
+        else if (t == "mix.q") rc = hy_place(s, l.win, s->Dp, 0, head_rows(d.heads, d.dim, rh, 0), s->D, f);
+        else if (t == "mix.k") rc = hy_place(s, l.win, s->Dp, 0, head_rows(kvh, d.dim, rh, l.e_q), s->D, f);
+        else if (t == "mix.v") rc = hy_place(s, l.win, s->Dp, 0, head_rows(kvh, d.vdim, 0, l.e_k), s->D, f);
+        else if (t == "mix.g") rc = hy_place(s, l.win, s->Dp, 0, head_rows(d.heads, d.vdim, 0, l.e_v), s->D, f);
+        else if (t == "mix.o") rc = hy_place(s, l.wout, l.Kp, 0, strided_rows(s->D, 0, 1), l.mixw, f);
+        else if (t == "mlp.gate") rc = hy_place(s, l.win, s->Dp, 0, strided_rows(d.ff, 2 * l.u1p, 2), s->D, f);
+        else if (t == "mlp.up") rc = hy_place(s, l.win, s->Dp, 0, strided_rows(d.ff, 2 * l.u1p + 1, 2), s->D, f);
+        else if (t == "mlp.down") rc = hy_place(s, l.wout, l.Kp, l.KA, strided_rows(s->D, 0, 1), d.ff, f);
         else {
             float* p = t == "mix.r1" ? l.r1 : t == "mix.r2" ? l.r2 : l.sink;
             SLI_HIP(hipMemcpy(p, host, sizeof(float) * n, hipMemcpyHostToDevice));
@@ -429,36 +441,39 @@ int hy_set_tensor(BlockStack* s, const std::string& name, const float* host, int
     return rc;
 }
 
+int hy_set_tensor(BlockStack* s, const std::string& name, const float* host, int64_t n) {
+    HyFill f;
+    f.host = host;
+    return hy_put(s, name, f, n);
+}
+
+// seeded random weights (matrices on the device)
 int hy_init_synthetic(BlockStack* s, uint32_t seed) {
     std::vector<std::string> names;
     for (auto& kv : s->want) names.push_back(kv.first);
-    std::vector<float> buf, block(1 << 20);
-    uint64_t st = 0x9E3779B97F4A7C15ull * (seed + 1);
-    auto rnd = [&]() {  // xorshift*, uniform in (-1, 1)
-        st ^= st >> 12, st ^= st << 25, st ^= st >> 27;
-        return (float)((double)((st * 0x2545F4914F6CDD1Dull) >> 40) / 8388608.0 - 1.0);
-    };
-    for (float& f : block) f = rnd();
+    uint32_t id = 0;
     for (const std::string& name : names) {
         int li;
         std::string t;
         int64_t rows, cols;
         hy_shape(s, name, &li, &t, &rows, &cols);
         const int64_t n = rows * cols;
-        buf.resize(n);
-        const bool gain = t == "norm1" || t == "norm2" || t == "final.norm";
-        const float a = gain ? 0.1f : t == "mix.r2" ? 0.2f : rows == 1 ? 1.0f
-                        : t == "canon1" || t == "canon2" ? 0.3f : t == "embed" ? 1.0f : 1.5f / std::sqrt((float)cols);
-        const float off = gain ? 1.0f : t == "mix.r2" ? 0.25f : rows == 1 ? 1.0f : 0.0f;
-        // one random block, read from a random offset per row (large matrices fill at memory speed)
-        for (int64_t i = 0; i < n;) {
-            st ^= st >> 12, st ^= st << 25, st ^= st >> 27;
-            const size_t o = (size_t)((st * 0x2545F4914F6CDD1Dull) >> 45) & ((1 << 19) - 1);
-            const int64_t c = std::min<int64_t>(std::min<int64_t>(n - i, 1 << 19), std::max<int64_t>(cols, 1));
-            for (int64_t j = 0; j < c; ++j) buf[i + j] = off + a * block[o + j];
-            i += c;
+        const bool canon = t == "canon1" || t == "canon2", gain = t == "norm1" || t == "norm2" || t == "final.norm";
+        HyFill f;
+        f.rand.seed = (seed * 0x9E3779B9u) ^ (++id * 0x85EBCA6Bu);
+        f.rand.amp = canon ? 0.3f : t == "embed" ? 1.0f : rows > 1 ? 1.5f / std::sqrt((float)cols) : 1.0f;
+        std::vector<float> v;
+        if (rows == 1 || canon) {
+            const float amp = gain ? 0.1f : t == "mix.r2" ? 0.2f : f.rand.amp;
+            const float off = gain ? 1.0f : t == "mix.r2" ? 0.25f : canon ? 0.0f : 1.0f;
+            uint64_t x = 0x9E3779B97F4A7C15ull * (f.rand.seed + 1ull);
+            for (int64_t i = 0; i < n; ++i) {
+                x ^= x >> 12, x ^= x << 25, x ^= x >> 27;
+                v.push_back(off + amp * (float)((double)((x * 0x2545F4914F6CDD1Dull) >> 40) / 8388608.0 - 1.0));
+            }
+            f.host = v.data();
         }
-        HY_TRY(hy_set_tensor(s, name, buf.data(), n));
+        HY_TRY(hy_put(s, name, f, n));
     }
     return SLI_OK;
 }

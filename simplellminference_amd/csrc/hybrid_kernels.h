@@ -253,13 +253,25 @@ __global__ void __launch_bounds__(256) hy_keys_kernel(const float* __restrict__ 
 
 // ---------------------------------------------------------------- weights
 // rows of a source matrix [nrows][ncols] into rows map[r] of a fused matrix (row stride ld), from column col0 on
-template <typename WT>
+struct HySrcBuf {
+    const float* p;
+    __device__ float operator()(size_t i) const { return p[i]; }
+};
+struct HySrcRand {  // uniform in (-amp, amp) by element index
+    uint32_t seed;
+    float amp;
+    __device__ float operator()(size_t i) const {
+        uint32_t h = (uint32_t)i * 2654435761u ^ (uint32_t)(i >> 32) * 0x9E3779B9u ^ seed;
+        h ^= h >> 16, h *= 0x7feb352du, h ^= h >> 15, h *= 0x846ca68bu, h ^= h >> 16;
+        return amp * ((float)(h >> 8) * (1.0f / 8388608.0f) - 1.0f);
+    }
+};
+template <typename WT, class Src>
 __global__ void __launch_bounds__(256) hy_place_kernel(WT* __restrict__ dst, int ld, int col0,
-                                                       const int32_t* __restrict__ map, int ncols,
-                                                       const float* __restrict__ src) {
+                                                       const int32_t* __restrict__ map, int ncols, Src src) {
     const int r = blockIdx.x;
     WT* d = dst + (size_t)map[r] * ld + col0;
-    for (int c = threadIdx.x; c < ncols; c += 256) d[c] = from_f32<WT>(src[(size_t)r * ncols + c]);
+    for (int c = threadIdx.x; c < ncols; c += 256) d[c] = from_f32<WT>(src((size_t)r * ncols + c));
 }
 
 }  // namespace sli
