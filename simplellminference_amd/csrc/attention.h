@@ -51,7 +51,8 @@ struct AttnArgs {
     // packed rows (attn_mfma.h ROWS): sequence i of the launch uses cache slot slot_dev[i * pos_seq_stride] (< 0: none),
     // with a distance bias r1 ln(1 + r2 distance) per query head of a sequence
     const int32_t* slot_dev = nullptr;
-    const float *bias_r1 = nullptr, *bias_r2 = nullptr;
+    const float *bias_r1 = nullptr, *bias_r2 = nullptr, *sink = nullptr;
+    int out_ld = 0, vdim = 0;        // out [sequences of the launch][out_ld], vdim dims per query head
     int* hand_err = nullptr;         // DevState::error: a bounded wait that gave up sets kAttnErrHand
 };
 

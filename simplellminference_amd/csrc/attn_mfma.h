@@ -115,8 +115,11 @@ __device__ __forceinline__ void am_split3(float v, __half& hi, __half& mid, __ha
 // sums), loading all of them in ONE batch of 16-byte o and 8-byte (m, l) write-through copies (sc1; 16 splits
 // per thread: ns <= 32 in one round trip), and the pair combines over DPP (lanes 2j, 2j+1). Deterministic: a
 // fixed split-to-thread map and combine order.
-template <int HD, int G, int NSH>
-__device__ __forceinline__ void am_merge(const float* part, float* out, int kvh, int max_splits, int ns) {
+// sink / vdim (packed rows): per query head of the kv head, exp(sink) joins the denominator, and out holds vdim <= HD
+// dims per query head; null / HD: neither.
+template <int HD, int G, int NSH, bool ROWS = false>
+__device__ __forceinline__ void am_merge(const float* part, float* out, int kvh, int max_splits, int ns,
+                                         const float* sink = nullptr, int vdim = HD) {
     constexpr int PS = HD + kAttnPartPad, NOG = G * HD / 4, NTH = 64 * kAmWaves, NPASS = (2 * NOG + NTH - 1) / NTH;
     const unsigned bytes = (unsigned)(sizeof(float) * (size_t)G * max_splits * PS);
     const auto rs = __builtin_amdgcn_make_buffer_rsrc(const_cast<float*>(part + (size_t)kvh * G * max_splits * PS), 0,
@@ -167,6 +170,18 @@ __device__ __forceinline__ void am_merge(const float* part, float* out, int kvh,
         const float Le = half ? Lp : L, Lo = half ? L : Lp;
         const float Lt = fmaf(ce, Le, co * Lo);
         const int ogv = (int)(threadIdx.x >> 1) + pass * (NTH / 2);
+        if constexpr (ROWS) {
+            const float sk = sink[g], Ms = fmaxf(Mt, sk), cm = expf(Mt - Ms), Ls = fmaf(cm, Lt, expf(sk - Ms));
+            if (half == 0 && ogv < NOG) {
+                const float y[4] = {fmaf(ce, oe.x, co * oo.x) * cm / Ls, fmaf(ce, oe.y, co * oo.y) * cm / Ls,
+                                    fmaf(ce, oe.z, co * oo.z) * cm / Ls, fmaf(ce, oe.w, co * oo.w) * cm / Ls};
+                float* dst = out + (size_t)g * vdim + d;
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (d + e < vdim) dst[e] = y[e];
+            }
+            continue;
+        }
         if (half == 0 && ogv < NOG)
             *reinterpret_cast<float4*>(out + (size_t)kvh * G * HD + (size_t)g * HD + d) =
                 make_float4(fmaf(ce, oe.x, co * oo.x) / Lt, fmaf(ce, oe.y, co * oo.y) / Lt,
@@ -177,8 +192,9 @@ __device__ __forceinline__ void am_merge(const float* part, float* out, int kvh,
 // grid: n_kv_heads (every sequence's) * max_splits workgroups of 256 threads; a.ppwg = kAmWgKeys * tpw (the
 // split length), NBUF = min(tpw, 2) ring slots per wave. The K/V rows of a split are read once (clamped to pos:
 // rows past the live context re-read row pos, an L2 hit, and are masked).
-// ROWS: packed rows (AttnArgs slot_dev, the distance bias); the split partials are always left to a merge that adds
-// the sink (attn_rows.h attn_sink_merge_kernel).
+// ROWS: packed rows (AttnArgs slot_dev, the distance bias). The splits are merged with the sink by the head's last
+// arriver into out [rows][out_ld] (vdim dims per query head), or (defer_merge) left to attn_rows.h
+// attn_sink_merge_kernel.
 template <int HD, int G, int NBUF, bool ROWS = false>
 __global__ void __launch_bounds__(64 * kAmWaves) attn_mfma_kernel(AttnArgs<__half> a) {
     using Geo = AmGeo<HD, G>;
@@ -396,7 +412,7 @@ __global__ void __launch_bounds__(64 * kAmWaves) attn_mfma_kernel(AttnArgs<__hal
         w4[w] = m4[w] == -INFINITY ? 0.0f : expf(m4[w] - M);
         L = fmaf(w4[w], reinterpret_cast<const float*>(sm + w * WB)[NT * 256 + 64 + lane], L);
     }
-    const bool publish = !ROWS && a.defer_merge == 0;
+    const bool publish = a.defer_merge == 0;
     for (int t = wave; t < NT; t += kAmWaves) {
         am_float4 acc = am_float4{0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
@@ -433,14 +449,23 @@ __global__ void __launch_bounds__(64 * kAmWaves) attn_mfma_kernel(AttnArgs<__hal
     }
     __syncthreads();
     if (last) {
+        float* out = a.out;
+        const float* sink = nullptr;
+        int vdim = HD;
+        if constexpr (ROWS) {
+            const int seq = kvh / a.seq_heads, qh = (kvh - seq * a.seq_heads) * G;
+            sink = a.sink + qh;
+            vdim = a.vdim;
+            out += (size_t)seq * a.out_ld + (size_t)qh * vdim;
+        }
         if (ns <= 4)
-            am_merge<HD, G, 2>(a.part, a.out, kvh, a.max_splits, ns);
+            am_merge<HD, G, 2, ROWS>(a.part, out, kvh, a.max_splits, ns, sink, vdim);
         else if (ns <= 8)
-            am_merge<HD, G, 4>(a.part, a.out, kvh, a.max_splits, ns);
+            am_merge<HD, G, 4, ROWS>(a.part, out, kvh, a.max_splits, ns, sink, vdim);
         else if (ns <= 16)
-            am_merge<HD, G, 8>(a.part, a.out, kvh, a.max_splits, ns);
+            am_merge<HD, G, 8, ROWS>(a.part, out, kvh, a.max_splits, ns, sink, vdim);
         else
-            am_merge<HD, G, 16>(a.part, a.out, kvh, a.max_splits, ns);
+            am_merge<HD, G, 16, ROWS>(a.part, out, kvh, a.max_splits, ns, sink, vdim);
         if (a.stamps && threadIdx.x == 0) a.stamps[blockIdx.x * 4 + 3] = __builtin_amdgcn_s_memrealtime();
     }
 }

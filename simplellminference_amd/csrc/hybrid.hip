@@ -13,6 +13,7 @@
 #include "attn_mfma.h"
 #include "attn_rows.h"
 #include "canon.h"
+#include "hybrid_gemv.h"
 #include "hybrid_kernels.h"
 #include "retention.h"
 #include "retention_chunk.h"
@@ -78,7 +79,9 @@ struct BlockStack {
     int32_t *nsegs = nullptr, *widx = nullptr;
     float *x = nullptr, *q = nullptr, *k = nullptr, *v = nullptr, *g = nullptr, *o = nullptr, *lg = nullptr;
     void *c1 = nullptr, *c2 = nullptr, *xl = nullptr;  // fp32 or fp16 by path
+    float* ssq = nullptr;    // retention: sums of o^2 per (head, slice) of a batch-1 step
     float* part = nullptr;   // split partials of the decode attention
+    unsigned* attn_cnt = nullptr;  // its per-head arrival counters (zero between launches)
     float* bg_ws = nullptr;  // split-K partials and arrival counters of the batched projections
     unsigned* bg_cnt = nullptr;
     std::vector<void*> allocs;
@@ -273,15 +276,19 @@ int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out)
     HY_TRY(hy_alloc(s, (void**)&s->g, sizeof(float) * M * nv));
     HY_TRY(hy_alloc(s, (void**)&s->o, sizeof(float) * M * no));
     HY_TRY(hy_alloc(s, (void**)&s->lg, sizeof(float) * M * s->V));
+    size_t nssq = 0;
+    for (const HyLayer& l : s->layers) nssq = std::max(nssq, (size_t)l.d.heads * l.nsl);
+    HY_TRY(hy_alloc(s, (void**)&s->ssq, sizeof(float) * nssq));
     const int Bp = s->B <= kBgMaxBatch ? s->B : pad_to(s->B, kHyTile);
-    size_t part = 0, bgp = 0, bgc = 1;
+    size_t part = 0, ncnt = 0, bgp = 0, bgc = 1;
     for (const HyLayer& l : s->layers) {
         if (l.d.mixer == SLI_MIX_ATTENTION)
-            part = std::max(part, (size_t)Bp * l.d.heads * hy_attn_splits(s->T) * (l.hd + kAttnPartPad));
-        if (s->f16 && s->B > 1)
+            part = std::max(part, (size_t)Bp * l.d.heads * hy_attn_splits(s->T) * (l.hd + kAttnPartPad)),
+            ncnt = std::max(ncnt, (size_t)Bp * l.d.heads);
+        if (s->f16)
             for (auto [np, K] : {std::make_pair(l.e_g, s->Dp), std::make_pair((int)l.d.ff, s->Dp),
                                  std::make_pair((s->D + 1) / 2, l.Kp), std::make_pair((s->V + 1) / 2, s->Dp)})
-                for (int b = 2; b <= std::min(s->B, kBgMaxBatch); ++b) {
+                for (int b = 2; b <= kBgMaxBatch; ++b) {  // (the head takes any number of wanted rows)
                     if (np == 0) continue;
                     const BgPlan p = bg_plan((np + 7) / 8, K, b, false, gemv_max_blocks());
                     SLI_CHECK(p.groups > 0, SLI_ERR_SHAPE, "stack: no tiling of a batched projection fits");
@@ -290,6 +297,7 @@ int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out)
                 }
     }
     HY_TRY(hy_alloc(s, (void**)&s->part, sizeof(float) * part));
+    HY_TRY(hy_alloc(s, (void**)&s->attn_cnt, sizeof(unsigned) * ncnt));
     HY_TRY(hy_alloc(s, (void**)&s->bg_ws, bgp + 256));
     HY_TRY(hy_alloc(s, (void**)&s->bg_cnt, sizeof(unsigned) * bgc));
     return hy_allow_lds();
@@ -678,6 +686,14 @@ struct HyRec {
                 a.scale = d.scale;
                 a.bias_r1 = l.r1;
                 a.bias_r2 = l.r2;
+                a.sink = l.sink;
+                a.counters = s->attn_cnt;
+                a.vdim = d.vdim;
+                a.out_ld = l.Kp;
+                if constexpr (std::is_same<OT, float>::value)
+                    a.out = l.cat32;
+                else
+                    a.defer_merge = 2;
                 const int tpw = attn_mfma_tpw(nkv, s->T, device_cus());
                 a.ppwg = kAmWgKeys * tpw;
                 a.max_splits = (s->T + a.ppwg - 1) / a.ppwg;
@@ -687,6 +703,7 @@ struct HyRec {
                 else
                     attn_split<128>(a, g, nkv * a.max_splits, tpw > 1);
                 SLI_HIP(hipGetLastError());
+                if (a.defer_merge == 0) return SLI_OK;  // merged into out by the launch itself
                 hipLaunchKernelGGL(attn_sink_merge_kernel<OT>, dim3(d.heads, M), dim3(128), 0, st(), s->part, ra,
                                    a.max_splits, a.ppwg, cat<OT>(l), l.Kp);
                 SLI_HIP(hipGetLastError());
@@ -717,9 +734,39 @@ struct HyRec {
             if (M > kBgMaxBatch) return layer_as<__half>(r);
         return layer_as<float>(r);
     }
+    // Batch 1: the layer as three launches (hybrid_gemv.h), where its shape fits their prologues
+    bool fits_fused(const HyLayer& l) const {
+        const sli_block_desc& d = l.d;
+        if (M != 1 || !one || s->taps != kCanonFusedTaps || s->Dp > 4 * kGemvThreads) return false;
+        if (!hy_out_fits(l.KA, l.KF, l.mixw, d.vdim)) return false;
+        return d.mixer == SLI_MIX_RETENTION || (F16 && l.hd <= 128);
+    }
+    int layer_fused(const HyRun& r) const {
+        const HyLayer& l = s->layers[r.layer];
+        const sli_block_desc& d = l.d;
+        SLI_HIP((launch_hy_in<WT>((const WT*)l.win, canon(l, r), in_epi<float>(l, r), l.e_g, l.u1p, (int)d.ff, st())));
+        HyOutIn o{};
+        o.cat = l.cat32;
+        o.KA = l.KA, o.KF = l.KF, o.mixw = l.mixw, o.vdim = d.vdim;
+        o.o = s->o, o.gate = s->g, o.ssq = s->ssq, o.nsl = l.nsl;
+        o.eps = s->c.eps;
+        const EpiStore<1> e{s->x, s->x, nullptr, s->c.residual_mult, s->D};
+        if (d.mixer == SLI_MIX_ATTENTION) {
+            HY_TRY(attention<float>(l, r));
+            SLI_HIP((launch_hy_out<WT, false>((const WT*)l.wout, o, e, s->D, st())));
+        } else {
+            RetArgs a{s->q, s->k, s->v, r.S, s->o, l.decay, s->rows, s->segs, s->nsegs, d.heads, d.dim, d.vdim, l.nsl};
+            a.ssq = s->ssq;
+            hipLaunchKernelGGL(ret_step_kernel, dim3(l.nsl, d.heads, 1), dim3(256), 0, st(), a);
+            SLI_HIP(hipGetLastError());
+            SLI_HIP((launch_hy_out<WT, true>((const WT*)l.wout, o, e, s->D, st())));
+        }
+        return SLI_OK;
+    }
     template <typename OT>
     int layer_as(const HyRun& r) const {
         const HyLayer& l = s->layers[r.layer];
+        if (fits_fused(l)) return layer_fused(r);
         const CanonArgs ca = canon(l, r);
         hipLaunchKernelGGL(canon_rows_kernel<OT>, dim3(M), dim3(256), 0, st(), ca, (OT*)s->c1,
                            l.d.ff > 0 ? (OT*)s->c2 : (OT*)nullptr, one ? 1 : 0);

@@ -844,7 +844,21 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
             x1[t] = pa_tr_read(a1 + ((c ^ s1) * 16));
             x2[t] = pa_tr_read(a2 + ((c ^ s2) * 16));
         }
-        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        // the transposed reads landed: their registers are named in the wait, so the MFMAs that use them stay below it
+        // (as in attn_mfma.h; an asm load's outputs count as written at its end)
+        if constexpr (NT == 8)
+            asm volatile("s_waitcnt lgkmcnt(0)"
+                         : "+v"(x1[0]), "+v"(x1[1]), "+v"(x1[2]), "+v"(x1[3]), "+v"(x1[4]), "+v"(x1[5]), "+v"(x1[6]),
+                           "+v"(x1[7]), "+v"(x2[0]), "+v"(x2[1]), "+v"(x2[2]), "+v"(x2[3]), "+v"(x2[4]), "+v"(x2[5]),
+                           "+v"(x2[6]), "+v"(x2[7])
+                         :
+                         : "memory");
+        else
+            asm volatile("s_waitcnt lgkmcnt(0)"
+                         : "+v"(x1[0]), "+v"(x1[1]), "+v"(x1[2]), "+v"(x1[3]), "+v"(x2[0]), "+v"(x2[1]), "+v"(x2[2]),
+                           "+v"(x2[3])
+                         :
+                         : "memory");
 #pragma unroll
         for (int t = 0; t < NT; ++t) {
             o[t] *= corr;

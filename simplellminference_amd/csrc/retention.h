@@ -27,6 +27,7 @@ struct RetArgs {
     const SegRef* segs;  // portions of the pass (scan / chunk forms)
     const int32_t* nsegs;
     int H, dim, vdim, nsl;
+    float* ssq = nullptr;  // [M][H][nsl] sums of o^2 over a slice (step form, nullable)
 };
 
 __device__ __forceinline__ float* ret_slice(const RetArgs& a, int slot, int h, int sl) {
@@ -89,6 +90,9 @@ __global__ void __launch_bounds__(256) ret_step_kernel(RetArgs a) {
         if (col + 1 < a.vdim) o[col + 1] = t.y;
         if (col + 2 < a.vdim) o[col + 2] = t.z;
         if (col + 3 < a.vdim) o[col + 3] = t.w;
+        // (columns past vdim are zero: their v is)
+        const float q2 = group_sum<8>(sq4(t));
+        if (a.ssq && c4 == 0) a.ssq[((size_t)m * a.H + h) * a.nsl + sl] = q2;
     }
 }
 
