@@ -184,7 +184,7 @@ inline bool hy_out_fits(int KA, int KF, int mixw, int vdim) {
 template <typename WT, bool RET>
 hipError_t launch_hy_out(const WT* W, const HyOutIn& a, const EpiStore<1>& e, int rows, hipStream_t s) {
     GemvIn in{nullptr, nullptr, 0.0f, a.KA + a.KF};
-    constexpr int U = 6, waves = kGemvThreads / 64;
+    constexpr int U = 4, waves = kGemvThreads / 64;
     const int cpr = (in.cols / Vec16<WT>::N + 64 * U - 1) / (64 * U);
     int cs = 1;
     while (cs < 8 && 2 * cs <= cpr && rows * cs < gemv_max_blocks() * waves) cs *= 2;
