@@ -15,7 +15,7 @@
 
 namespace sli {
 
-constexpr int kHyMaxRows = 512;  // rows of one pass
+constexpr int kHyMaxRows = 1024;  // rows of one pass
 constexpr int kHyTile = 32;      // a portion's rows start at a multiple of this (one sequence per row tile)
 
 struct BlockStack;

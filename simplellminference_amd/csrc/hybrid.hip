@@ -26,6 +26,7 @@ namespace sli {
         if (rc_ != SLI_OK) return rc_; \
     } while (0)
 
+constexpr int kHyLogitRows = 256;  // wanted rows per pass of the output head
 constexpr int kHySection = 128;  // pairs: a GEMM row block (at most 256 rows) never straddles the two inputs
 
 static int pad_to(int n, int m) { return (n + m - 1) / m * m; }
@@ -275,7 +276,7 @@ int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out)
     HY_TRY(hy_alloc(s, (void**)&s->v, sizeof(float) * M * nv));
     HY_TRY(hy_alloc(s, (void**)&s->g, sizeof(float) * M * nv));
     HY_TRY(hy_alloc(s, (void**)&s->o, sizeof(float) * M * no));
-    HY_TRY(hy_alloc(s, (void**)&s->lg, sizeof(float) * M * s->V));
+    HY_TRY(hy_alloc(s, (void**)&s->lg, sizeof(float) * kHyLogitRows * s->V));
     size_t nssq = 0;
     for (const HyLayer& l : s->layers) nssq = std::max(nssq, (size_t)l.d.heads * l.nsl);
     HY_TRY(hy_alloc(s, (void**)&s->ssq, sizeof(float) * nssq));
@@ -568,7 +569,7 @@ struct HyRec {
         if constexpr (F16) {
             PgIn<__half> in{w, X, nullptr, pad_to(2 * npairs, 16), K, M};
             if (X2) in.Bhi2 = X2, in.row_b2 = 2 * split;
-            return pg_pick(M, [&](auto cfg) -> int {
+            return pg_pick(M, in.N, [&](auto cfg) -> int {
                 SLI_HIP((launch_pgemm<PgPair<Epi>, decltype(cfg), __half>(in, PgPair<Epi>{e, npairs, u0}, nullptr, st())));
                 return SLI_OK;
             });
@@ -576,17 +577,24 @@ struct HyRec {
             return fail(SLI_ERR_ARG, "prompt GEMM: fp16 weights");
         }
     }
+    // Tilings (their row count divides M) by rows and output tiles, the fastest of a sweep at 4096 x 15104 and 34304 x 4096 with the weights streamed
+    // from HBM (TFLOP/s at 1024 rows 794 and 814, at 512 591 and 658, at 256 296 and 579): one 256 x 256 tile per CU
+    // where the grid fills the chip with them, smaller tiles (a full grid) where the output is narrow.
     template <class F>
-    static int pg_pick(int M, F&& f) {
-        if (M % 128 == 0) return f(PgCfg<128, 2, 3, 4, true, 0, 1>{});
+    static int pg_pick(int M, int N, F&& f) {
+        const long long t128 = (long long)((N + 127) / 128) * (M / 128);
+        if (M % 256 == 0 && M != 512 && t128 >= 512) return f(PgCfg<256, 4, 2, 4, true, 0, 1>{});
+        if (M % 128 == 0 && M >= 512 && t128 >= 512) return f(PgCfg<128, 4, 2, 2, true, 0, 1>{});
+        if (M % 128 == 0 && t128 >= 256) return f(PgCfg<128, 2, 3, 4, true, 0, 1>{});
+        if (M % 64 == 0 && M >= 128) return f(PgCfg<64, 4, 4, 2, true, 0, 1>{});
         if (M % 64 == 0) return f(PgCfg<64, 2, 4, 2, true, 0, 1>{});
         return f(PgCfg<32, 2, 4, 2, true, 0, 1>{});
     }
     template <class Epi>
     static int allow() {
         if constexpr (F16) {
-            for (int M : {32, 64, 128})
-                HY_TRY(pg_pick(M, [&](auto cfg) -> int {
+            for (auto [M, N] : {std::make_pair(32, 128), {64, 128}, {128, 128}, {128, 1 << 15}, {256, 1 << 15}, {512, 1 << 15}})
+                HY_TRY(pg_pick(M, N, [&](auto cfg) -> int {
                     SLI_HIP((pgemm_allow_lds<PgPair<Epi>, decltype(cfg), __half>()));
                     return SLI_OK;
                 }));
@@ -917,8 +925,12 @@ int hy_pass(BlockStack* s, const std::vector<RowRef>& rows_in, const std::vector
     if (!want.empty()) {
         const int nw = (int)want.size();
         SLI_HIP(hipMemcpyAsync(s->widx, want.data(), sizeof(int32_t) * nw, hipMemcpyHostToDevice, s->stream));
-        HY_TRY(HY_DISPATCH(s, M, one, msegs, logits(s->widx, nw, s->lg)));
-        SLI_HIP(hipMemcpyAsync(logits_host, s->lg, sizeof(float) * (size_t)nw * s->V, hipMemcpyDeviceToHost, s->stream));
+        for (int w = 0; w < nw; w += kHyLogitRows) {
+            const int n = std::min(kHyLogitRows, nw - w);
+            HY_TRY(HY_DISPATCH(s, M, one, msegs, logits(s->widx + w, n, s->lg)));
+            SLI_HIP(hipMemcpyAsync(logits_host + (size_t)w * s->V, s->lg, sizeof(float) * (size_t)n * s->V,
+                                   hipMemcpyDeviceToHost, s->stream));
+        }
     }
     SLI_HIP(hipStreamSynchronize(s->stream));
     return SLI_OK;

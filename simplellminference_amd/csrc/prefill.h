@@ -583,6 +583,7 @@ struct PgEpiResid {  // y[m][row] = resid[m][row] + sum * row scale (matmul_kern
 template <class Epi, class Cfg, typename WT>
 hipError_t launch_pgemm(const PgIn<WT>& in, const Epi& epi, const PfState* ps, hipStream_t s) {
     using Geo = PgGeo<Cfg, WT>;
+    if (in.M % Geo::BM != 0) return hipErrorInvalidValue;  // rows past the last whole tile would be skipped
     const int nrb = (in.N + Geo::BN - 1) / Geo::BN;
     const int nrb8 = (nrb + 7) / 8 * 8;
     const dim3 grid(nrb8 * (in.M / Geo::BM));

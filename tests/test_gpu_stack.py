@@ -201,6 +201,21 @@ def test_portions_of_a_prompt(gpu, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+def test_wide_projections(gpu, dtype):
+    """Feed-forward and output head wide enough for every GEMM tiling, in passes of 1024, 512, 256, 128 and 96 rows and
+    with wanted-row counts that are no multiple of a tile."""
+    c = stack(ret(ff=8300), att(ff=40), width=64, vocab=1001)
+    t = R.random_tensors(c, 23)
+    ids = tokens(1060, c["vocab"], 24)
+    want = R.forward(c, t, ids)[0]
+    m = make(c, t, dtype, 1100)
+    close(pieces(m, ids, []), want, dtype, "whole")
+    for cut in ([500, 720, 830, 920], [213, 300, 400, 550]):
+        close(pieces(m, ids, cut), want, dtype, f"cut {cut}")
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("lens", [(5, 70, 33), (1, 2, 3, 130, 64, 31, 32, 97), tuple(range(3, 14))])
 def test_batches_of_unequal_requests(gpu, lens, dtype):
     """Prompts as one batch, decoded together, the shorter ones ending earlier: each as it is alone."""

@@ -207,8 +207,8 @@ def _cfg():
 FAULTS = {
     "sink": lambda mp, c, t: t.update({"l1.mix.sink": t["l1.mix.sink"] - 50.0}),
     "bias": lambda mp, c, t: t.update({"l1.mix.r1": 0 * t["l1.mix.r1"]}),
-    "bias distance off by one": lambda mp, c, t: mp.setattr(
-        R, "attention_weights", lambda q, k, s, r1, r2, sk, f=R.attention_weights: f(q, k, s, r1, 0.5 * r2, sk)),
+    "bias distance": lambda mp, c, t: mp.setattr(
+        R, "attention_weights", lambda q, k, s, r1, r2, sk, f=R.attention_weights: f(q, k, s, r1, 5.0 * r2, sk)),
     "decay": lambda mp, c, t: c["blocks"][0].update(decay=(0.75, 0.93)),
     "rotation base": lambda mp, c, t: c["blocks"][0].update(rot_base=140.0),
     "rotation dims": lambda mp, c, t: c["blocks"][0].update(rot_dims=6),
@@ -220,8 +220,8 @@ FAULTS = {
     "clamp": lambda mp, c, t: c["blocks"][1].update(ff_limit=1.3),
     "head mapping": lambda mp, c, t: t.update({"l1.mix.k": np.roll(t["l1.mix.k"], 16, 0)}),
     "loop": lambda mp, c, t: c.update(loop=(0, 1, 1)),
-    "residual": lambda mp, c, t: c.update(residual_mult=0.42),
-    "embedding scale": lambda mp, c, t: c.update(emb_scale=1.6),
+    "residual": lambda mp, c, t: c.update(residual_mult=0.5),
+    "embedding scale": lambda mp, c, t: c.update(emb_scale=3.0),
 }
 
 
