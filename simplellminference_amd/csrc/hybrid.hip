@@ -289,7 +289,7 @@ int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out)
         if (s->f16)
             for (auto [np, K] : {std::make_pair(l.e_g, s->Dp), std::make_pair((int)l.d.ff, s->Dp),
                                  std::make_pair((s->D + 1) / 2, l.Kp), std::make_pair((s->V + 1) / 2, s->Dp)})
-                for (int b = 2; b <= kBgMaxBatch; ++b) {  // (the head takes any number of wanted rows)
+                for (int b = 1; b <= kBgMaxBatch; ++b) {  // (the head takes any number of wanted rows)
                     if (np == 0) continue;
                     const BgPlan p = bg_plan((np + 7) / 8, K, b, false, gemv_max_blocks());
                     SLI_CHECK(p.groups > 0, SLI_ERR_SHAPE, "stack: no tiling of a batched projection fits");
@@ -525,14 +525,14 @@ struct HyRec {
     int msegs;  // portions at most
     hipStream_t st() const { return s->stream; }
 
-    // How a projection over M rows runs: the batch-1 GEMV, the batched MFMA projection (2 .. 8 rows), the prompt GEMM
-    // (fp16, more rows), or the plain kernel (fp32, more than one row; widths past the GEMV's LDS stage).
+    // How a projection over M rows runs: the batch-1 GEMV, the batched MFMA projection (fp16, 2 .. 8 rows; one row past
+    // the GEMV's LDS stage), the prompt GEMM (fp16, more rows), or the plain kernel (fp32, more rows or wider).
     enum Path { GV, BG, PG, RG };
     static constexpr bool F16 = std::is_same<WT, __half>::value;
     static Path path(int M, int K) {
         if (M == 1 && K <= kGemvMaxCols) return GV;
         if (!F16) return RG;
-        return M <= kBgMaxBatch ? (M == 1 ? RG : BG) : PG;
+        return M <= kBgMaxBatch ? BG : PG;
     }
     // rows of the launches for n rows
     static int rows_for(int n) { return F16 && n > kBgMaxBatch ? pad_to(n, kHyTile) : n; }
@@ -623,6 +623,7 @@ struct HyRec {
         e.hd = l.hd, e.T = s->T;
         e.kscale = (float)(1.0 / std::sqrt((double)d.dim));
         e.limit = d.ff_limit;
+        e.even = d.dim % 4 == 0 && d.vdim % 4 == 0 && e.rh % 2 == 0;
         if (l.rot >= 0) e.cs = s->rots[l.rot].cs, e.sn = s->rots[l.rot].sn;
         e.q = l.q ? l.q : s->q, e.k = s->k, e.v = s->v, e.g = s->g;
         e.kc = (KT*)r.kc, e.vc = (KT*)r.vc;
@@ -776,9 +777,7 @@ struct HyRec {
         const HyLayer& l = s->layers[r.layer];
         if (fits_fused(l)) return layer_fused(r);
         const CanonArgs ca = canon(l, r);
-        hipLaunchKernelGGL(canon_rows_kernel<OT>, dim3(M), dim3(256), 0, st(), ca, (OT*)s->c1,
-                           l.d.ff > 0 ? (OT*)s->c2 : (OT*)nullptr, one ? 1 : 0);
-        SLI_HIP(hipGetLastError());
+        SLI_HIP((launch_canon_rows<OT>(ca, (OT*)s->c1, l.d.ff > 0 ? (OT*)s->c2 : (OT*)nullptr, one ? 1 : 0, st())));
         if (!one) {
             hipLaunchKernelGGL(canon_ring_kernel, dim3(M), dim3(256), 0, st(), ca);
             SLI_HIP(hipGetLastError());
@@ -832,7 +831,7 @@ struct HyRec {
         return SLI_OK;
     }
     int step(const DevState* dst, int B, float* y, unsigned long long* keys, int key_ld, int* nkeys) const {
-        hipLaunchKernelGGL(hy_rows_kernel, dim3(1), dim3(64), 0, st(), dst, s->rows, B, M);
+        hipLaunchKernelGGL(hy_rows_kernel, dim3(1), dim3(256), 0, st(), dst, s->rows, B, M);
         SLI_HIP(hipGetLastError());
         HY_TRY(pass());
         if (B == 1 && path(1, s->Dp) == GV) {
@@ -845,9 +844,9 @@ struct HyRec {
             return SLI_OK;
         }
         HY_TRY(logits(nullptr, B, y));
-        hipLaunchKernelGGL(hy_keys_kernel, dim3(B), dim3(256), 0, st(), y, s->V, keys, key_ld);
+        *nkeys = std::max(1, std::min({key_ld, 64, s->V / 1024}));
+        hipLaunchKernelGGL(hy_keys_kernel, dim3(B, *nkeys), dim3(256), 0, st(), y, s->V, keys, key_ld);
         SLI_HIP(hipGetLastError());
-        *nkeys = 1;
         return SLI_OK;
     }
     static int allow_all() {
@@ -861,6 +860,8 @@ struct HyRec {
 static int hy_allow_lds() {
     SLI_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(&ret_chunk_kernel<256>),
                                 hipFuncAttributeMaxDynamicSharedMemorySize, (int)RcGeo<256>::LDS));
+    SLI_HIP(hy_out_allow_lds<__half>());
+    SLI_HIP(hy_out_allow_lds<float>());
     return HyRec<__half>::allow_all();
 }
 

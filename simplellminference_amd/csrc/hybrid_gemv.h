@@ -178,7 +178,23 @@ __global__ void __launch_bounds__(kGemvThreads) hy_out_kernel(const WT* __restri
 }
 
 inline bool hy_out_fits(int KA, int KF, int mixw, int vdim) {
-    return KA + KF <= kGemvMaxCols && KA <= 4 * kGemvThreads && KF <= 4 * kGemvThreads * kHyOutAct && vdim % 4 == 0 && mixw >= 4;
+    return KA <= 4 * kGemvThreads && KF <= 4 * kGemvThreads * kHyOutAct && vdim % 4 == 0 && mixw >= 4;
+}
+
+// (the widest input, 20480 columns, takes more LDS than a launch gets by default)
+template <typename WT>
+hipError_t hy_out_allow_lds() {
+    hipError_t r = hipSuccess;
+    auto allow = [&](auto* k) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                                 160 * 1024);
+        if (e != hipSuccess) r = e;
+    };
+    allow(&hy_out_kernel<WT, true, 4, true>);
+    allow(&hy_out_kernel<WT, true, 4, false>);
+    allow(&hy_out_kernel<WT, false, 4, true>);
+    allow(&hy_out_kernel<WT, false, 4, false>);
+    return r;
 }
 
 template <typename WT, bool RET>

@@ -19,11 +19,8 @@ namespace sli {
 // rows of a decode step from the engine's states: one row per slot
 // (rows B .. M - 1: padding)
 __global__ void hy_rows_kernel(const DevState* st, RowRef* rows, int B, int M) {
-    const int b = threadIdx.x;
-    if (b < B)
-        rows[b] = RowRef{b, st[b].pos, st[b].token, b};
-    else if (b < M)
-        rows[b] = RowRef{-1, 0, 0, b};
+    for (int b = threadIdx.x; b < M; b += blockDim.x)
+        rows[b] = b < B ? RowRef{b, st[b].pos, st[b].token, b} : RowRef{-1, 0, 0, b};
 }
 
 template <typename WT>
@@ -39,6 +36,11 @@ __global__ void __launch_bounds__(256) hy_embed_kernel(const RowRef* __restrict_
 }
 
 // ---------------------------------------------------------------- epilogues: pair(u, m, v0, v1)
+// (pair2: pairs u and u + 1 at once, u even)
+__device__ __forceinline__ void store2(float* p, const float* v) { *reinterpret_cast<float2*>(p) = make_float2(v[0], v[1]); }
+__device__ __forceinline__ void store2(__half* p, const float* v) {
+    *reinterpret_cast<__half2*>(p) = __halves2half2(__float2half_rn(v[0]), __float2half_rn(v[1]));
+}
 // The fused input projection. Pairs [0, e_g): the mixer's q, k, v(, g) heads; pairs [u1p, u1p + ff): {gate, up}.
 // OT: element type of the feed-forward product in the output projection's input.
 template <typename KT, typename OT>
@@ -55,6 +57,56 @@ struct HyIn {
     OT* act;
     int act_ld, act_off;
     const RowRef* rows;
+    int even;                        // dim, vdim multiples of 4, rh even: two neighbouring pairs share a head and a branch
+    __device__ float glu(float gate, float up) const {
+        const float gt = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+        return gt / (1.0f + expf(-1.702f * gt)) * (u + 1.0f);
+    }
+    // pairs u and u + 1, u even: one row lookup and one head division, neighbouring results stored together
+    __device__ void pair2(int u, int m, const float* a, bool second) const {
+        if (!even || !second || (u < u1p ? u + 1 >= e_g : u + 1 - u1p >= ff)) {
+            pair(u, m, a[0], a[1]);
+            if (second) pair(u + 1, m, a[2], a[3]);
+            return;
+        }
+        const RowRef r = rows[m];
+        if (r.slot < 0) return;
+        if (u >= u1p) {
+            const float y[2] = {glu(a[0], a[1]), glu(a[2], a[3])};
+            store2(act + (size_t)m * act_ld + act_off + (u - u1p), y);
+            return;
+        }
+        const bool qk = u < e_k, isq = u < e_q, isv = u < e_v;
+        const int uu = isq ? u : qk ? u - e_q : isv ? u - e_k : u - e_v;
+        const int hp = qk ? hpq : hpv, h = uu / hp, j = uu - h * hp;
+        if (qk && j < rh) {  // two rotation pairs {j, j + rh}, {j + 1, j + 1 + rh} (retention only)
+            const size_t at = (size_t)r.pos * rh + j;
+            const float c0 = cs[at], s0 = sn[at], c1 = cs[at + 1], s1 = sn[at + 1], f = isq ? 1.0f : kscale;
+            float* p = (isq ? q : k) + ((size_t)m * H + h) * dim + j;
+            const float lo[2] = {(a[0] * c0 - a[1] * s0) * f, (a[2] * c1 - a[3] * s1) * f};
+            const float hi[2] = {(a[1] * c0 + a[0] * s0) * f, (a[3] * c1 + a[2] * s1) * f};
+            store2(p, lo);
+            store2(p + rh, hi);
+            return;
+        }
+        if (!retention) {
+            if (isq) {
+                *reinterpret_cast<float4*>(q + ((size_t)m * H + h) * hd + 2 * j) = make_float4(a[0], a[1], a[2], a[3]);
+            } else {
+                KT* p = (qk ? kc : vc) + (((size_t)r.slot * G + h) * T + r.pos) * hd + 2 * j;
+                store2(p, a);
+                store2(p + 2, a + 2);
+            }
+            return;
+        }
+        float4 y = make_float4(a[0], a[1], a[2], a[3]);
+        if (qk && !isq) y = make_float4(y.x * kscale, y.y * kscale, y.z * kscale, y.w * kscale);
+        if (!isv)
+            y = make_float4(y.x / (1.0f + expf(-y.x)), y.y / (1.0f + expf(-y.y)), y.z / (1.0f + expf(-y.z)),
+                            y.w / (1.0f + expf(-y.w)));
+        float* p = isq ? q : qk ? k : isv ? v : g;
+        *reinterpret_cast<float4*>(p + ((size_t)m * H + h) * (qk ? dim : vdim) + 2 * j) = y;
+    }
     __device__ void dims(int j, int n, int& d0, int& d1) const {  // pair j of a head of n dims (d1 < 0: none)
         if (j < rh) {
             d0 = j, d1 = j + rh;
@@ -69,9 +121,7 @@ struct HyIn {
         if (u >= u1p) {
             const int i = u - u1p;
             if (i >= ff) return;
-            const float gt = fminf(a0, limit), up = fminf(fmaxf(a1, -limit), limit);
-            const float y = gt / (1.0f + expf(-1.702f * gt)) * (up + 1.0f);
-            act[(size_t)m * act_ld + act_off + i] = from_f32<OT>(y);
+            act[(size_t)m * act_ld + act_off + i] = from_f32<OT>(glu(a0, a1));
             return;
         }
         if (u >= e_g) return;
@@ -133,6 +183,17 @@ struct HyOut {
         if (2 * u < D) p[0] = fmaf(mult, v0, p[0]);
         if (2 * u + 1 < D) p[1] = fmaf(mult, v1, p[1]);
     }
+    __device__ void pair2(int u, int m, const float* a, bool) const {  // u even, ld a multiple of 4
+        float* p = x + (size_t)m * ld + 2 * u;
+        if (2 * u + 3 < D) {
+            const float4 r = *reinterpret_cast<const float4*>(p);
+            *reinterpret_cast<float4*>(p) =
+                make_float4(fmaf(mult, a[0], r.x), fmaf(mult, a[1], r.y), fmaf(mult, a[2], r.z), fmaf(mult, a[3], r.w));
+            return;
+        }
+        pair(u, m, a[0], a[1]);
+        pair(u + 1, m, a[2], a[3]);
+    }
 };
 
 struct HyLogits {
@@ -143,6 +204,10 @@ struct HyLogits {
         float* p = y + (size_t)m * n + 2 * u;
         if (2 * u < n) p[0] = v0;
         if (2 * u + 1 < n) p[1] = v1;
+    }
+    __device__ void pair2(int u, int m, const float* a, bool) const {
+        pair(u, m, a[0], a[1]);
+        pair(u + 1, m, a[2], a[3]);
     }
 };
 
@@ -183,8 +248,7 @@ struct PgPair {  // prefill.h: plain 16-row tiles, 4 consecutive rows per store
     __device__ int row(int t, int i) const { return t * 16 + i; }
     __device__ void store(int t, int i0, int m, const float* v, const PfState*) const {
         const int u = t * 8 + (i0 >> 1);
-        if (u < n) e.pair(u0 + u, m, v[0], v[1]);
-        if (u + 1 < n) e.pair(u0 + u + 1, m, v[2], v[3]);
+        if (u < n) e.pair2(u0 + u, m, v, u + 1 < n);
     }
 };
 
@@ -238,7 +302,7 @@ __global__ void __launch_bounds__(256) hy_keys_kernel(const float* __restrict__ 
     __shared__ unsigned long long red[4];
     const float* y = logits + (size_t)blockIdx.x * n;
     unsigned long long b = 0;
-    for (int i = threadIdx.x; i < n; i += 256) {
+    for (int i = blockIdx.y * 256 + threadIdx.x; i < n; i += 256 * gridDim.y) {
         const unsigned long long k = argmax_key(y[i], (unsigned)i);
         b = k > b ? k : b;
     }
@@ -247,7 +311,7 @@ __global__ void __launch_bounds__(256) hy_keys_kernel(const float* __restrict__ 
     __syncthreads();
     if (threadIdx.x == 0) {
         for (int w = 1; w < 4; ++w) b = red[w] > b ? red[w] : b;
-        keys[(size_t)blockIdx.x * key_ld] = red[0] > b ? red[0] : b;
+        keys[(size_t)blockIdx.x * key_ld + blockIdx.y] = red[0] > b ? red[0] : b;
     }
 }
 

@@ -3,7 +3,7 @@
 //   S  <- decay^n S + sum_j decay^(n-1-j) k_j v_j^T                               (n tokens in the chunk)
 // A workgroup of 4 waves owns one (portion, head, kRetCols value columns) and walks the portion's chunks. The state
 // slice stays in fp32 accumulators (C tiles of the update's own MFMAs) from the first chunk to the last, so it is never
-// rounded; where it is an operand (S^T q) it is carried as fp16 hi + lo, like the decayed scores and the decayed keys.
+// rounded; where it is an operand (S^T q) it is carried as fp16 hi + lo, like the decayed scores and the decayed values.
 // q, k and v enter as fp16. Operands reach their MFMA layouts through LDS; the next chunk's rows are loaded while the
 // current one is computed.
 #pragma once
@@ -17,13 +17,23 @@ constexpr int kRcTok = 32;
 template <int KD>  // dim padded to a multiple of 32
 struct RcGeo {
     static constexpr int QS = KD + 8, TS = kRcTok + 8;  // LDS row strides in halves (16-byte aligned, spread over banks)
-    static constexpr int Q = 0, K = Q + kRcTok * QS, KT = K + kRcTok * QS, KTL = KT + KD * TS, VT = KTL + KD * TS,
-                         ST = VT + kRetCols * TS, STL = ST + kRetCols * QS, P = STL + kRetCols * QS, PL = P + kRcTok * TS,
+    static constexpr int Q = 0, K = Q + kRcTok * QS, KT = K + kRcTok * QS, VT = KT + KD * TS,
+                         VD = VT + kRetCols * TS, VDL = VD + kRetCols * TS, ST = VDL + kRetCols * TS, STL = ST + kRetCols * QS, P = STL + kRetCols * QS, PL = P + kRcTok * TS,
                          END = PL + kRcTok * TS;
     static constexpr size_t LDS = (size_t)END * 2 + 4 * 64;  // + decay powers
     static constexpr int NT = KD / 16;                     // 16-row state tiles (x 2 column tiles)
     static constexpr int TPW = (NT * 2 + 3) / 4;           // state tiles per wave
     static constexpr int VEC = kRcTok * KD / 4 / 256;      // float4 of q (and of k) per thread per chunk
+    // piece i of thread tid: token and first dim (tokens 2p, 2p + 1 of one dim group are pieces of one thread: their
+    // transposed copies are one 4-byte store)
+    static constexpr int TOKS = VEC >= 2 ? 2 : 1;
+    __device__ static void piece(int i, int tid, int& t, int& d) {
+        const int e = (i / TOKS) * 256 + tid;
+        t = TOKS * (e / (KD / 4)) + i % TOKS;
+        d = 4 * (e % (KD / 4));
+    }
+    // K^T: the 8-token blocks of row d permuted by d / 16, so that the lanes of a transposed store spread over the banks
+    __device__ static int kt(int d, int t) { return KT + d * TS + ((t >> 3) ^ ((d >> 4) & 3)) * 8 + (t & 7); }
 };
 
 template <int KD>
@@ -61,7 +71,8 @@ __global__ void __launch_bounds__(256) ret_chunk_kernel(RetArgs a) {
         const bool al = a.dim % 4 == 0;
 #pragma unroll
         for (int i = 0; i < G::VEC; ++i) {
-            const int e = (i * 256 + tid) * 4, t = e / KD, d = e - t * KD;
+            int t, d;
+            G::piece(i, tid, t, d);
             const bool ok = c0 + t < sg.n;
             const size_t row = ((size_t)(sg.row0 + c0 + (ok ? t : 0)) * a.H + h) * a.dim;
             if (al) {
@@ -93,23 +104,34 @@ __global__ void __launch_bounds__(256) ret_chunk_kernel(RetArgs a) {
         __syncthreads();  // the previous chunk's LDS reads are done (first chunk: pw is there)
 #pragma unroll
         for (int i = 0; i < G::VEC; ++i) {
-            const int e = (i * 256 + tid) * 4, t = e / KD, d = e - t * KD;
+            int t, d;
+            G::piece(i, tid, t, d);
             store4(sm + G::Q + t * G::QS + d, qr[i]);
             store4(sm + G::K + t * G::QS + d, kr[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < G::VEC; i += G::TOKS) {
+            int t, d;
+            G::piece(i, tid, t, d);
             const float f[4] = {kr[i].x, kr[i].y, kr[i].z, kr[i].w};
-            const float w = pw[max(n - 1 - t, 0)];  // (rows past the portion are zero)
+            const float4& k1 = kr[i + G::TOKS - 1];
+            const float f1[4] = {k1.x, k1.y, k1.z, k1.w};
 #pragma unroll
             for (int x = 0; x < 4; ++x) {
-                __half hi, lo;
-                pf_split(f[x] * w, hi, lo);
-                sm[G::KT + (d + x) * G::TS + t] = hi;
-                sm[G::KTL + (d + x) * G::TS + t] = lo;
+                if constexpr (G::TOKS == 2)
+                    *reinterpret_cast<__half2*>(sm + G::kt(d + x, t)) = __halves2half2(__float2half_rn(f[x]), __float2half_rn(f1[x]));
+                else
+                    sm[G::kt(d + x, t)] = __float2half_rn(f[x]);
             }
         }
 #pragma unroll
         for (int i = 0; i < NV; ++i) {
             const int e = i * 256 + tid, t = e / kRetCols, c = e % kRetCols;
             sm[G::VT + c * G::TS + t] = __float2half_rn(vr[i]);
+            __half hi, lo;
+            pf_split(vr[i] * pw[max(n - 1 - t, 0)], hi, lo);  // (rows past the portion are zero)
+            sm[G::VD + c * G::TS + t] = hi;
+            sm[G::VDL + c * G::TS + t] = lo;
         }
         // the state before this chunk, as the S^T q operand [column][row]
 #pragma unroll
@@ -155,9 +177,9 @@ __global__ void __launch_bounds__(256) ret_chunk_kernel(RetArgs a) {
             const int t = wave * G::TPW + i;
             if (t < 2 * G::NT) {
                 st[i] *= dn;
-                const u32x4 v = frag(G::VT, (t % 2) * 16 + i16, G::TS, 0);
-                st[i] = pf_mfma(frag(G::KT, (t / 2) * 16 + i16, G::TS, 0), v, st[i]);
-                st[i] = pf_mfma(frag(G::KTL, (t / 2) * 16 + i16, G::TS, 0), v, st[i]);
+                const u32x4 kt = *reinterpret_cast<const u32x4*>(sm + G::kt((t / 2) * 16 + i16, 8 * g));
+                st[i] = pf_mfma(kt, frag(G::VD, (t % 2) * 16 + i16, G::TS, 0), st[i]);
+                st[i] = pf_mfma(kt, frag(G::VDL, (t % 2) * 16 + i16, G::TS, 0), st[i]);
             }
         }
         __syncthreads();

@@ -216,6 +216,41 @@ def test_wide_projections(gpu, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+def test_long_output_rows(gpu, dtype):
+    """An output projection whose input [mixer; feed-forward] is longer than 16384: with and without the shapes that the
+    fused batch-1 launches take, alone and as a batch."""
+    c = stack(att(ff=16300), ret(vdim=33, ff=16370), ret(vdim=32, ff=16384), width=32, vocab=61)
+    t = R.random_tensors(c, 25)
+    a, b = tokens(45, c["vocab"], 26), tokens(45, c["vocab"], 27)
+    want = [R.forward(c, t, i)[0] for i in (a, b)]
+    m = make(c, t, dtype, 64, batch=2)
+    close(pieces(m, a, range(1, 45)), want[0], dtype, "token by token")
+    m.feed([0, 1], [0, 0], [a[:40], b[:40]])
+    for p in range(40, 45):
+        got = m.feed([0, 1], [p, p], [[a[p]], [b[p]]], [[0], [0]])
+        close(got, np.stack([w[p] for w in want]), dtype, f"batch, position {p}")
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_many_sequences_in_lockstep(gpu, dtype):
+    """The engine's own batched step over the most sequences it takes, teacher-forced."""
+    t = R.random_tensors(PAIR, 28)
+    n = 64
+    ids = [tokens(6, PAIR["vocab"], 100 + i) for i in range(n)]
+    m = make(PAIR, t, dtype, 16, batch=n)
+    lg = np.empty((6, n, PAIR["vocab"]), np.float32)
+    for p in range(6):
+        for i in range(n):
+            m.set_state_seq(i, ids[i][p], p, advance=False)
+        m.step()
+        lg[p] = m.logits()[0]
+    for i in (0, 1, 31, 32, 62, 63):
+        close(lg[:, i], R.forward(PAIR, t, ids[i])[0], dtype, f"sequence {i}")
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("lens", [(5, 70, 33), (1, 2, 3, 130, 64, 31, 32, 97), tuple(range(3, 14))])
 def test_batches_of_unequal_requests(gpu, lens, dtype):
     """Prompts as one batch, decoded together, the shorter ones ending earlier: each as it is alone."""
