@@ -101,8 +101,10 @@ class StackModel(LlamaModel):
     def _load_weights(self) -> "StackModel":
         if self.model_path:
             st = SafeTensors(os.path.join(self.model_path, "model.safetensors"))
-            for name in st.names():
-                self.set_tensor(name, st.get(name))
+            unused = {f"l{i}.{n}" for i, b in enumerate(self.spec.blocks) if not b.ff for n in ("norm2", "canon2")}
+            for name in st.names():  # (a block without a feed-forward may still name its second sublayer's norm and taps)
+                if name not in unused:
+                    self.set_tensor(name, st.get(name))
         elif self.seed is not None:
             call("sli_model_init_synthetic", self._h, self.seed)
         return self
