@@ -455,6 +455,20 @@ def test_folder_trace_and_command_line(gpu, dtype, tmp_path, capsys, monkeypatch
         assert outs[0] == outs[1]
 
 
+def test_folder_without_a_feed_forward(gpu, tmp_path):
+    """A null feed-forward, with and without the second sublayer's norm and taps in the file."""
+    from simplellminference_amd.registry import load_model
+    c = stack(att(ff=0), ret(ff=24), width=40)
+    t = bf16(R.random_tensors(c, 29))
+    ids = tokens(20, c["vocab"], 30)
+    want = R.forward(c, t, ids)[0]
+    for extra in ({}, {"l0.norm2": np.float64(3.0), "l0.canon2": np.ones((40, 4))}):
+        rugudra_folder(tmp_path, c, {**t, **extra})
+        m = load_model(str(tmp_path), "float32", 32)
+        close(m.feed([0], [0], [ids], [list(range(20))]), want, "float32")
+        m.close()
+
+
 def test_errors_come_from_the_host(gpu):
     from simplellminference_amd._lib import SliError
     t = R.random_tensors(PAIR, 24)
