@@ -287,27 +287,43 @@ int sli_tp_group_predict_prefill(sli_tp_group* g, const int32_t* prompt, int32_t
                                  int32_t* tokens_out, float* logits_out);
 
 /* ---------------------------------------------------------------- block-stack models
- * A decoder described by data, behind the same sli_model handle and decode loop as the Llama models: n_blocks
- * parallel blocks x += residual_mult * (mixer(c1) + ff(c2)), c1 / c2 = the RMS-normed rows (one gain per sublayer)
- * after a causal per-channel convolution of `taps` taps that is added to its input; blocks loop_start ..
- * loop_stop - 1 run loop_times times in a row (same weights, one cache or state per run).
+ * A decoder described by data, behind the same sli_model handle and decode loop as the Llama models. x = embed[token]
+ * emb_scale (+ a learned row per position where `positions` > 0); n_blocks blocks, run in the order of `runs` (n_runs
+ * block indices; null: in order, blocks loop_start .. loop_stop - 1 loop_times times in a row) with the block's weights
+ * and one cache or state per run. Two arrangements:
+ *
+ * SLI_STACK_PARALLEL: x += residual_mult * (mixer(c1) + ff(c2)), c1 / c2 = the RMS-normed rows (one gain per sublayer)
+ * after a causal per-channel convolution of `taps` taps that is added to its input. Mixers: attention, retention;
+ * dense feed-forward.
+ *
+ * SLI_STACK_SEQUENTIAL: x += norm1(rg1 * mixer(c)), then x += norm2(rg2 * ff(x)): the norms (one gain per channel) are on
+ * the sublayers' outputs, c = x after the input convolution, and rg = sigmoid(W x + b) gates each output element by
+ * element (x as the sublayer found it). Mixer: latent attention; feed-forward: a mixture of experts, or none.
+ *
  * Mixers: SLI_MIX_ATTENTION, causal grouped-query softmax attention without rotation, scores (q . k) * scale
  * - r1 ln(1 + r2 distance) and a sink per head; SLI_MIX_RETENTION, linear attention with a fixed decay per head
  * (decay: the retention blocks' values, concatenated in block order), rotate-half positions on the first rot_dims
- * dims, the output normalised per head and gated by silu. Feed-forward (ff > 0): g = min(gate, ff_limit),
- * u = clamp(up, +-ff_limit), down(g sigmoid(1.702 g) (u + 1)).
+ * dims, the output normalised per head and gated by silu. SLI_MIX_LATENT, softmax attention without positions whose
+ * keys and values are projections of one cached RMS-normed row of kv_rank values per token, over the last `window`
+ * positions (0: all), scores (q . k) * scale, the output gated by a sigmoid projection of the mixer's input.
+ * Feed-forward (ff > 0): dense (experts 0): g = min(gate, ff_limit), u = clamp(up, +-ff_limit), down(g sigmoid(1.702 g)
+ * (u + 1)). Mixture (experts > 0): `top` of `experts` experts silu(gate) * up -> down of ff rows, chosen by the largest
+ * router logits and weighted by the softmax over the chosen ones.
  * Weights: SLI_DT_F16 (bfloat16 checkpoints: every bfloat16 value of magnitude 2^-14 .. 65504 is kept exactly) with
  * an fp16 cache, or SLI_DT_F32 with an fp32 cache (true fp32 throughout). Norms, convolutions, scores, softmax,
  * recurrent state and residual are fp32 in both. */
-typedef enum { SLI_MIX_ATTENTION = 0, SLI_MIX_RETENTION = 1 } sli_mixer_kind;
+typedef enum { SLI_MIX_ATTENTION = 0, SLI_MIX_RETENTION = 1, SLI_MIX_LATENT = 2 } sli_mixer_kind;
+typedef enum { SLI_STACK_PARALLEL = 0, SLI_STACK_SEQUENTIAL = 1 } sli_stack_arrangement;
 typedef struct {
     int32_t mixer; /* sli_mixer_kind */
     int32_t heads, kv_heads, dim, vdim;
-    float scale;      /* attention */
+    float scale;      /* attention, latent attention */
     int32_t rot_dims; /* retention */
     double rot_base;
-    int32_t ff;       /* 0: no feed-forward */
-    float ff_limit;
+    int32_t ff;       /* rows of the feed-forward (of each expert); 0: no feed-forward */
+    float ff_limit;   /* dense */
+    int32_t kv_rank, window; /* latent attention */
+    int32_t experts, top;    /* mixture (0: dense) */
 } sli_block_desc;
 typedef struct {
     int32_t vocab, width, n_blocks, loop_start, loop_stop, loop_times, taps;
@@ -316,10 +332,16 @@ typedef struct {
     const float* decay;
     int32_t w_dtype; /* SLI_DT_F16 or SLI_DT_F32 */
     int32_t max_len, batch, device;
+    int32_t arrangement; /* sli_stack_arrangement */
+    int32_t positions;   /* rows of the learned position table; 0: none (else max_len is at most this) */
+    const int32_t* runs; /* nullable */
+    int32_t n_runs;
 } sli_stack_config;
 int sli_stack_create(const sli_stack_config* cfg, sli_model** out);
-/* One tensor as full fp32 [n]: embed, head, final.norm, l<i>.{norm1,norm2,canon1,canon2}, l<i>.mix.{q,k,v,o} and
- * {r1,r2,sink} (attention) or {g} (retention), l<i>.mlp.{gate,up,down}; matrices [out][in]. */
+/* One tensor as full fp32 [n], block i's as l<i>.*; matrices [out][in]. embed, head, final.norm, pos (positions);
+ * parallel: norm1, norm2, canon1, canon2, mix.{q,k,v,o} and {r1,r2,sink} (attention) or {g} (retention),
+ * mlp.{gate,up,down}; sequential: norm1, norm2, canon1, rg1, rg1.b, rg2, rg2.b, mix.{q,dkv,dkv.norm,uk,uv,g,o},
+ * mlp.{router,router.b}, mlp.e<j>.{gate,up,down}. */
 int sli_stack_set_tensor(sli_model* m, const char* name, const float* host, int64_t n);
 /* Feed the next tokens of n sequences as one batch: sequence slot slots[i] gets lens[i] tokens (concatenated in
  * `tokens`) from position starts[i] on (0: a new sequence, whatever the slot held; else the position its earlier

@@ -44,14 +44,16 @@ class ShardWindow(ctypes.Structure):
 
 class BlockDesc(ctypes.Structure):
     _fields_ = [(n, c_i32) for n in ("mixer", "heads", "kv_heads", "dim", "vdim")] + \
-               [("scale", c_f), ("rot_dims", c_i32), ("rot_base", c_d), ("ff", c_i32), ("ff_limit", c_f)]
+               [("scale", c_f), ("rot_dims", c_i32), ("rot_base", c_d), ("ff", c_i32), ("ff_limit", c_f)] + \
+               [(n, c_i32) for n in ("kv_rank", "window", "experts", "top")]
 
 
 class StackConfig(ctypes.Structure):
     _fields_ = [(n, c_i32) for n in ("vocab", "width", "n_blocks", "loop_start", "loop_stop", "loop_times", "taps")] + \
                [(n, c_f) for n in ("eps", "emb_scale", "residual_mult")] + \
                [("blocks", ctypes.POINTER(BlockDesc)), ("decay", P_f)] + \
-               [(n, c_i32) for n in ("w_dtype", "max_len", "batch", "device")]
+               [(n, c_i32) for n in ("w_dtype", "max_len", "batch", "device", "arrangement", "positions")] + \
+               [("runs", P_i32), ("n_runs", c_i32)]
 
 
 # name -> (restype, argtypes)

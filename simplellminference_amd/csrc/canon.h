@@ -6,7 +6,7 @@
 // a sublayer's gain and its "+ h_t" term are folded into its taps at load (c_t = sum_j f_j * n_(t-j), f_0 = g (1 +
 // w_last), f_j = g w_(last-j)), and ONE ring of past n rows per layer run and sequence slot is the state of both
 // convolutions: position p lives in ring row p % taps, so a decode step overwrites the row no tap reads any more.
-// Everything here is fp32.
+// Everything here is fp32. CanonArgs::raw: the same for a sublayer that reads the residual stream without a norm.
 #pragma once
 #include "common.h"
 #include "gemv.h"
@@ -25,6 +25,8 @@ struct CanonArgs {
     const RowRef* rows;   // [M]
     float eps;
     int D, ld, taps, M;
+    bool raw = false;     // no norm: h is the residual row itself (the ring holds x rows); c2, where given without f2, is
+                          // a copy of it
 };
 
 template <typename T>
@@ -72,7 +74,7 @@ __global__ void __launch_bounds__(256) canon_rows_kernel(CanonArgs a, OT* c1, OT
     __shared__ float inv[kCanonMaxTaps];
     const int nin = min(min(a.taps - 1, r.pos), m - r.first);  // earlier rows of this pass under the taps
     for (int j = 0; j <= nin; ++j) {
-        const float v = row_inv_rms(a.x + (size_t)(m - j) * a.ld, a.ld, a.D, a.eps, red);
+        const float v = a.raw ? 1.0f : row_inv_rms(a.x + (size_t)(m - j) * a.ld, a.ld, a.D, a.eps, red);
         if (threadIdx.x == 0) inv[j] = v;
     }
     __syncthreads();
@@ -88,6 +90,7 @@ __global__ void __launch_bounds__(256) canon_rows_kernel(CanonArgs a, OT* c1, OT
                 n = reinterpret_cast<const float4*>(ring + (size_t)((r.pos - j) % a.taps) * a.ld)[i];
             s1 = fma4(n, reinterpret_cast<const float4*>(a.f1 + (size_t)j * a.ld)[i], s1);
             if (a.f2) s2 = fma4(n, reinterpret_cast<const float4*>(a.f2 + (size_t)j * a.ld)[i], s2);
+            if (j == 0 && !a.f2) s2 = n;
             if (j == 0 && write_ring) reinterpret_cast<float4*>(ring + (size_t)(r.pos % a.taps) * a.ld)[i] = n;
         }
         store4(c1 + (size_t)m * a.ld + 4 * i, s1);
@@ -119,19 +122,21 @@ __global__ void __launch_bounds__(1024) canon4_rows_kernel(CanonArgs a, OT* c1, 
                                     : j <= nall ? ring + (size_t)((r.pos - j) % TAPS) * a.ld : a.x + (size_t)m * a.ld;
         n[j] = reinterpret_cast<const float4*>(src)[i];
         f1[j] = reinterpret_cast<const float4*>(a.f1 + (size_t)j * a.ld)[i];
-        f2[j] = reinterpret_cast<const float4*>((c2 ? a.f2 : a.f1) + (size_t)j * a.ld)[i];
+        f2[j] = reinterpret_cast<const float4*>((a.f2 ? a.f2 : a.f1) + (size_t)j * a.ld)[i];
     }
+    if (!a.raw) {
 #pragma unroll
-    for (int j = 0; j < TAPS; ++j) {
-        const float ss = wave_sum(tid < n4 ? sq4(n[j]) : 0.0f);
-        if ((tid & 63) == 0) red[tid >> 6][j] = ss;
+        for (int j = 0; j < TAPS; ++j) {
+            const float ss = wave_sum(tid < n4 ? sq4(n[j]) : 0.0f);
+            if ((tid & 63) == 0) red[tid >> 6][j] = ss;
+        }
+        __syncthreads();
     }
-    __syncthreads();
     float4 s1 = make_float4(0.f, 0.f, 0.f, 0.f), s2 = s1;
 #pragma unroll
     for (int j = TAPS - 1; j >= 0; --j) {
         if (j > nall) continue;
-        if (j <= nin) {
+        if (j <= nin && !a.raw) {
             float t = 0.0f;
             for (int w = 0; w < (int)blockDim.x / 64; ++w) t += red[w][j];
             n[j] = mul4(n[j], 1.0f / sqrtf(t / (float)a.D + a.eps));
@@ -142,7 +147,7 @@ __global__ void __launch_bounds__(1024) canon4_rows_kernel(CanonArgs a, OT* c1, 
     if (tid >= n4) return;
     if (write_ring) reinterpret_cast<float4*>(ring + (size_t)(r.pos % TAPS) * a.ld)[i] = n[0];
     store4(c1 + (size_t)m * a.ld + 4 * i, s1);
-    if (c2) store4(c2 + (size_t)m * a.ld + 4 * i, s2);
+    if (c2) store4(c2 + (size_t)m * a.ld + 4 * i, a.f2 ? s2 : n[0]);
 }
 
 template <typename OT>
@@ -155,14 +160,14 @@ hipError_t launch_canon_rows(const CanonArgs& a, OT* c1, OT* c2, int write_ring,
 }
 
 // the last min(n, taps - 1) rows of every portion into the ring (after canon_rows_kernel of the same pass)
-__global__ void __launch_bounds__(256) canon_ring_kernel(CanonArgs a) {
+static __global__ void __launch_bounds__(256) canon_ring_kernel(CanonArgs a) {
     __shared__ float red[4];
     const int m = blockIdx.x;
     const RowRef r = a.rows[m];
     if (r.slot < 0) return;
     const int later = m + a.taps - 1;  // a later row of the portion that far ahead: this row is out of every tap's reach
     if (later < a.M && a.rows[later].slot >= 0 && a.rows[later].first == r.first) return;
-    const float inv = row_inv_rms(a.x + (size_t)m * a.ld, a.ld, a.D, a.eps, red);
+    const float inv = a.raw ? 1.0f : row_inv_rms(a.x + (size_t)m * a.ld, a.ld, a.D, a.eps, red);
     float* ring = a.ring + ((size_t)r.slot * a.taps + r.pos % a.taps) * a.ld;
     for (int i = threadIdx.x; i < a.ld / 4; i += 256)
         reinterpret_cast<float4*>(ring)[i] = mul4(reinterpret_cast<const float4*>(a.x + (size_t)m * a.ld)[i], inv);

@@ -1983,6 +1983,7 @@ extern "C" int sli_model_feed(sli_model* m, int32_t n, const int32_t* slots, con
     std::vector<float> lbuf, hbuf;
     int i0 = 0;  // first entry with tokens left
     while (i0 < n) {
+        int kt = 0;  // expanded rows of the pass
         std::vector<RowRef> rows;
         std::vector<SegRef> segs;
         std::vector<int32_t> widx;
@@ -1996,6 +1997,11 @@ extern "C" int sli_model_feed(sli_model* m, int32_t n, const int32_t* slots, con
             }
             const int room = kHyMaxRows - (int)rows.size(), c = std::min(room, lens[i] - done[i]);
             if (c <= 0) break;
+            if (!one) {
+                const int t = hy_key_tiles(m->bs, starts[i] + done[i], c);
+                if (!segs.empty() && kt + t > hy_key_tiles_max(m->bs)) break;
+                kt += t;
+            }
             const int first = (int)rows.size();
             segs.push_back(SegRef{slots[i], first, c, starts[i] + done[i]});
             for (int j = 0; j < c; ++j) {

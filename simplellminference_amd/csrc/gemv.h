@@ -68,6 +68,17 @@ __host__ __device__ constexpr bool stage_late() {
     return StageLate<S>::value;
 }
 
+// Epilogues whose column parts are rows of their own (kParts = true, SPLIT only): unit u is the sum over csplit parts of
+// row rows_part(u, p) (cols columns each) times part p of the staged input [csplit][cols] (moe.h: one part per expert).
+template <class E, class = void>
+struct EpiParts {
+    static constexpr bool value = false;
+};
+template <class E>
+struct EpiParts<E, std::void_t<decltype(E::kParts)>> {
+    static constexpr bool value = E::kParts;
+};
+
 template <int G>
 struct XStage {
     float4 xr[kGemvStageV4];
@@ -366,7 +377,9 @@ __device__ __forceinline__ void gemv_block(const WT* __restrict__ W, const GemvI
     // cpp chunks; the workgroup's (unit, part) items are balanced over its waves and the parts' row sums
     // are added in part order in the epilogue. CS = 1: one item per unit, the whole row per wave.
     const int CS = SPLIT ? in.csplit : 1;  // compile-time 1 unless the launch split the columns
-    const int cpp = (cpr + CS - 1) / CS;  // chunks per part (a part past the row end is all masked)
+    constexpr bool PARTS = EpiParts<Epi>::value;
+    static_assert(!PARTS || SPLIT, "parts need the split form");
+    const int cpp = PARTS ? cpr : (cpr + CS - 1) / CS;  // chunks per part (a part past the row end is all masked)
     const int ni = (ue - ub) * CS;       // the workgroup's items
     // in.cw streaming waves share the items; a wave past them has none and repeats the loads of wave
     // (wave - cw)'s first steps (L2 hits on lines in flight), so no load sits behind a branch
@@ -376,7 +389,7 @@ __device__ __forceinline__ void gemv_block(const WT* __restrict__ W, const GemvI
     const int ib = (int)(((unsigned)wq * (unsigned)ni) / (unsigned)cw);
     const int ie = idle ? ib : (int)(((unsigned)(wq + 1) * (unsigned)ni) / (unsigned)cw);
     const int nsteps = (ie - ib) * cpp;
-    float* res = smem + kGemvLdsHead + in.cols;
+    float* res = smem + kGemvLdsHead + (PARTS ? in.cols * CS : in.cols);
 
     const unsigned long long t_entry = in.stamps ? __builtin_amdgcn_s_memrealtime() : 0;
     unsigned long long t_staged = 0;
@@ -409,8 +422,11 @@ __device__ __forceinline__ void gemv_block(const WT* __restrict__ W, const GemvI
     auto load_step = [&](const Pos& q, u32x4 (&w)[U][R]) {
         const Pos& a = q.it > it_last ? dummy : q;
         int rows[R];
-        epi.rows(min(a.u, nunits - 1), rows);
-        const int v = (a.p * cpp + a.cc) * CV + lane;
+        if constexpr (PARTS)
+            epi.rows_part(min(a.u, nunits - 1), a.p, rows);
+        else
+            epi.rows(min(a.u, nunits - 1), rows);
+        const int v = (PARTS ? a.cc : a.p * cpp + a.cc) * CV + lane;
 #pragma unroll
         for (int j = 0; j < U; ++j) {
             const int vj = min(v + j * 64, nvec - 1);  // clamp, never branch around a load
@@ -433,12 +449,13 @@ __device__ __forceinline__ void gemv_block(const WT* __restrict__ W, const GemvI
 #pragma unroll
     for (int r = 0; r < R; ++r) acc[r] = 0.0f;
     auto consume_step = [&](const Pos& q, const u32x4(&w)[U][R]) {
-        const int c = q.p * cpp + q.cc;
+        const int c = PARTS ? q.cc : q.p * cpp + q.cc;
         const int v = c * CV + lane;
+        const float* xp = PARTS ? xs + (size_t)q.p * in.cols : xs;
         if ((c + 1) * CV <= nvec)
-            gemv_chunk<WT, R, U>(w, xs, v, acc);
+            gemv_chunk<WT, R, U>(w, xp, v, acc);
         else
-            gemv_chunk<WT, R, U, true>(w, xs, v, acc, nvec);
+            gemv_chunk<WT, R, U, true>(w, xp, v, acc, nvec);
         if (q.cc == cpp - 1) {  // item complete: its R partial row sums go to LDS
 #pragma unroll
             for (int r = 0; r < R; ++r) {

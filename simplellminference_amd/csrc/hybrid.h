@@ -1,7 +1,8 @@
 // hybrid.h — block-stack models behind the engine's model handle (engine.hip): a decoder whose layers are described
-// by data (sli_stack_config, include/sli.h), each a parallel block x += mult * (mixer(c1) + ff(c2)) with an
-// attention or a retention mixer, an input convolution per sublayer (canon.h), and a range of layers that may run
-// several times with shared weights and one cache or state per run.
+// by data (sli_stack_config, include/sli.h), in one of two arrangements: parallel blocks x += mult * (mixer(c1) + ff(c2))
+// with an attention or a retention mixer (hybrid.hip), or sequential sublayers x += norm(gate * sublayer(x)) with latent
+// attention and a mixture of experts (hybrid_seq.hip); both with an input convolution (canon.h) and with blocks that may
+// run several times with shared weights and one cache or state per run.
 //
 // The engine keeps what every model has (device decode state, prompts, history, graphs, greedy sampling); this file's
 // functions are the forward pass over packed rows (step_state.h RowRef): a decode step has one row per sequence,
@@ -28,6 +29,10 @@ int hy_fill_context(BlockStack* s, uint32_t seed, int upto);
 // before a capture or an eager pass: every tensor is there, the folded coefficients and tables are uploaded
 int hy_prepare(BlockStack* s);
 int hy_runs(const BlockStack* s);
+// A prompt pass also expands cached rows (latent attention): what a portion of n tokens at pos0 adds, and the most a pass
+// may hold (one portion of kHyMaxRows rows always fits)
+int hy_key_tiles(const BlockStack* s, int pos0, int n);
+int hy_key_tiles_max(const BlockStack* s);
 
 // Decode step of every slot, from the engine's device states: embedding .. logits [B][V] and the argmax keys
 // (*nkeys per sequence at keys[b * key_ld]).

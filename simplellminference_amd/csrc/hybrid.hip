@@ -2,11 +2,9 @@
 // recorded launches of a decode step and of a prompt pass.
 #include "hybrid.h"
 
-#include <algorithm>
 #include <cmath>
 #include <cstdlib>
 #include <cstring>
-#include <map>
 #include <type_traits>
 
 #include "../../include/sli_synth.h"
@@ -15,82 +13,16 @@
 #include "canon.h"
 #include "hybrid_gemv.h"
 #include "hybrid_kernels.h"
+#include "hybrid_rec.h"
+#include "hybrid_stack.h"
+#include "latent.h"
 #include "retention.h"
 #include "retention_chunk.h"
 
 namespace sli {
 
-#define HY_TRY(expr)                   \
-    do {                               \
-        int rc_ = (expr);              \
-        if (rc_ != SLI_OK) return rc_; \
-    } while (0)
-
-constexpr int kHyLogitRows = 256;  // wanted rows per pass of the output head
-constexpr int kHySection = 128;  // pairs: a GEMM row block (at most 256 rows) never straddles the two inputs
-
-static int pad_to(int n, int m) { return (n + m - 1) / m * m; }
-
-struct HyLayer {
-    sli_block_desc d{};
-    int mixw = 0, KA = 0, KF = 0, Kp = 0;  // output projection input: [mixer (KA) ; feed-forward (KF)]
-    int hpq = 0, hpv = 0, e_q = 0, e_k = 0, e_v = 0, e_g = 0, u1p = 0, u2p = 0;
-    int hd = 0;   // attention: padded cache row
-    int nsl = 0;  // retention: state slices per head
-    int rot = -1;
-    void *win = nullptr, *wout = nullptr;
-    float *f1 = nullptr, *f2 = nullptr, *r1 = nullptr, *r2 = nullptr, *sink = nullptr, *decay = nullptr;
-    // the output projection's input and the attention query rows, one buffer per shape: their padding columns are never
-    // written, so they stay zero
-    float *cat32 = nullptr, *q = nullptr;
-    __half* cat16 = nullptr;
-    float n1 = 0.0f, n2 = 0.0f;
-    std::vector<float> c1, c2;  // [width][taps] as given
-};
-
-struct HyRun {
-    int layer = 0;
-    void *kc = nullptr, *vc = nullptr;
-    float *S = nullptr, *ring = nullptr;
-};
-
-struct HyRot {
-    int dims = 0;
-    double base = 0.0;
-    float *cs = nullptr, *sn = nullptr;
-};
-
-struct BlockStack {
-    sli_stack_config c{};
-    hipStream_t stream = nullptr;
-    bool f16 = true;
-    size_t wb = 2;
-    int D = 0, Dp = 0, V = 0, Vp = 0, T = 0, B = 0, taps = 0, M = 0;  // taps: padded tap count; M: rows of a pass
-    std::vector<HyLayer> layers;
-    std::vector<HyRun> runs;
-    std::vector<HyRot> rots;
-    void *emb = nullptr, *head = nullptr;
-    float *fnorm = nullptr, *fnorm_p = nullptr;  // final gain per channel; times sqrt(D / Dp)
-    float fgain = 0.0f;
-    std::map<std::string, bool> want;  // tensor -> placed
-    bool dirty = true;
-    // activations of a pass
-    RowRef* rows = nullptr;
-    SegRef* segs = nullptr;
-    int32_t *nsegs = nullptr, *widx = nullptr;
-    float *x = nullptr, *q = nullptr, *k = nullptr, *v = nullptr, *g = nullptr, *o = nullptr, *lg = nullptr;
-    void *c1 = nullptr, *c2 = nullptr, *xl = nullptr;  // fp32 or fp16 by path
-    float* ssq = nullptr;    // retention: sums of o^2 per (head, slice) of a batch-1 step
-    float* part = nullptr;   // split partials of the decode attention
-    unsigned* attn_cnt = nullptr;  // its per-head arrival counters (zero between launches)
-    float* bg_ws = nullptr;  // split-K partials and arrival counters of the batched projections
-    unsigned* bg_cnt = nullptr;
-    std::vector<void*> allocs;
-    std::vector<std::pair<hipGraph_t, hipGraphExec_t>> graphs_one, graphs_rows;
-};
-
 // ---------------------------------------------------------------- creation
-static int hy_alloc(BlockStack* s, void** p, size_t bytes, bool zero = true) {
+int hy_alloc(BlockStack* s, void** p, size_t bytes, bool zero) {
     bytes = std::max<size_t>(bytes, 16);
     hipError_t e = hipMalloc(p, bytes);
     if (e != hipSuccess) return hip_fail(e, "hipMalloc");
@@ -103,7 +35,9 @@ static int hy_layer_init(HyLayer& l, int i) {
     const sli_block_desc& d = l.d;
     const std::string at = "block " + std::to_string(i) + ": ";
     SLI_CHECK(d.heads > 0 && d.dim > 0 && d.vdim > 0 && d.ff >= 0, SLI_ERR_SHAPE, at + "non-positive size");
-    SLI_CHECK(d.mixer == SLI_MIX_ATTENTION || d.mixer == SLI_MIX_RETENTION, SLI_ERR_ARG, at + "unknown mixer");
+    SLI_CHECK(d.mixer == SLI_MIX_ATTENTION || d.mixer == SLI_MIX_RETENTION, SLI_ERR_ARG,
+              at + "a parallel block mixes with attention or retention");
+    SLI_CHECK(d.experts == 0 && d.window == 0, SLI_ERR_ARG, at + "a parallel block has no experts and no window");
     l.mixw = d.heads * d.vdim;
     l.KA = pad_to(l.mixw, 64);
     l.KF = pad_to(d.ff, 64);
@@ -142,28 +76,21 @@ static int hy_attn_splits(int T) { return std::max(kAmMaxSplits, (T + 64 * kAmWg
 
 static int hy_allow_lds();
 
-int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out) {
-    const sli_stack_config& c = *cfg;
-    SLI_CHECK(c.vocab > 0 && c.width > 0 && c.n_blocks > 0 && c.blocks && c.max_len > 0 && c.batch > 0, SLI_ERR_SHAPE,
-              "stack: non-positive dimension");
-    SLI_CHECK(c.taps >= 1 && c.taps <= kCanonMaxTaps, SLI_ERR_SHAPE, "stack: taps must be 1 .. 32");
-    SLI_CHECK(c.loop_start >= 0 && c.loop_start <= c.loop_stop && c.loop_stop <= c.n_blocks && c.loop_times >= 1,
-              SLI_ERR_SHAPE, "stack: bad loop");
-    SLI_CHECK(c.w_dtype == SLI_DT_F16 || c.w_dtype == SLI_DT_F32, SLI_ERR_ARG, "stack: fp16 or fp32 weights");
-    BlockStack* s = new BlockStack();
-    *out = s;  // destroyed by the caller on failure
-    s->c = c;
-    s->stream = stream;
-    s->f16 = c.w_dtype == SLI_DT_F16;
-    s->wb = s->f16 ? 2 : 4;
-    s->D = c.width;
-    s->Dp = pad_to(c.width, 64);
-    s->V = c.vocab;
-    s->Vp = pad_to(c.vocab, 128);
-    s->T = c.max_len;
-    s->B = c.batch;
-    s->taps = std::max(c.taps, kCanonFusedTaps);
-    s->M = kHyMaxRows;
+// the batched projections of np pairs over K columns: their workspace (every row count; the head takes any number of wanted rows)
+int hy_bg_need(BlockStack* s, int np, int K) {
+    if (!s->f16 || np == 0) return SLI_OK;
+    for (int b = 1; b <= kBgMaxBatch; ++b) {
+        const BgPlan p = bg_plan((np + 7) / 8, K, b, false, gemv_max_blocks());
+        SLI_CHECK(p.groups > 0, SLI_ERR_SHAPE, "stack: no tiling of a batched projection fits");
+        s->bg_ws_bytes = std::max(s->bg_ws_bytes, bg_part_bytes(p));
+        s->bg_groups = std::max(s->bg_groups, (size_t)p.groups);
+    }
+    return SLI_OK;
+}
+
+// layers, rotation tables and activations of the parallel arrangement
+static int par_create(BlockStack* s) {
+    const sli_stack_config& c = s->c;
     s->layers.resize(c.n_blocks);
     size_t nq = 0, nk = 0, nv = 0, no = 0;
     int dec = 0;
@@ -237,31 +164,93 @@ int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out)
         SLI_HIP(hipMemcpy(r.cs, cs.data(), sizeof(float) * cs.size(), hipMemcpyHostToDevice));
         SLI_HIP(hipMemcpy(r.sn, sn.data(), sizeof(float) * sn.size(), hipMemcpyHostToDevice));
     }
-    auto add_run = [&](int i) {
-        HyRun r;
-        r.layer = i;
-        s->runs.push_back(r);
-    };
-    for (int i = 0; i < c.loop_start; ++i) add_run(i);
-    for (int t = 0; t < c.loop_times; ++t)
-        for (int i = c.loop_start; i < c.loop_stop; ++i) add_run(i);
-    for (int i = c.loop_stop; i < c.n_blocks; ++i) add_run(i);
     for (HyRun& r : s->runs) {
         const HyLayer& l = s->layers[r.layer];
-        HY_TRY(hy_alloc(s, (void**)&r.ring, sizeof(float) * (size_t)s->B * s->taps * s->Dp));
+        HY_TRY(hy_new(s, &r.ring, (size_t)s->B * s->taps * s->Dp));
         if (l.d.mixer == SLI_MIX_ATTENTION) {
             const size_t n = (size_t)s->B * l.d.kv_heads * s->T * l.hd * (s->f16 ? 2 : 4);
             HY_TRY(hy_alloc(s, &r.kc, n));
             HY_TRY(hy_alloc(s, &r.vc, n));
         } else {
-            HY_TRY(hy_alloc(s, (void**)&r.S, sizeof(float) * (size_t)s->B * l.d.heads * l.nsl * l.d.dim * kRetCols));
+            HY_TRY(hy_new(s, &r.S, (size_t)s->B * l.d.heads * l.nsl * l.d.dim * kRetCols));
         }
     }
+    const size_t M = s->M;
+    HY_TRY(hy_new(s, &s->q, M * nq));
+    HY_TRY(hy_new(s, &s->k, M * nk));
+    HY_TRY(hy_new(s, &s->v, M * nv));
+    HY_TRY(hy_new(s, &s->g, M * nv));
+    HY_TRY(hy_new(s, &s->o, M * no));
+    size_t nssq = 0;
+    for (const HyLayer& l : s->layers) nssq = std::max(nssq, (size_t)l.d.heads * l.nsl);
+    HY_TRY(hy_new(s, &s->ssq, nssq));
+    const int Bp = s->B <= kBgMaxBatch ? s->B : pad_to(s->B, kHyTile);
+    size_t part = 0, ncnt = 0;
+    for (const HyLayer& l : s->layers) {
+        if (l.d.mixer == SLI_MIX_ATTENTION)
+            part = std::max(part, (size_t)Bp * l.d.heads * hy_attn_splits(s->T) * (l.hd + kAttnPartPad)),
+            ncnt = std::max(ncnt, (size_t)Bp * l.d.heads);
+        HY_TRY(hy_bg_need(s, l.e_g, s->Dp));
+        HY_TRY(hy_bg_need(s, l.d.ff, s->Dp));
+        HY_TRY(hy_bg_need(s, (s->D + 1) / 2, l.Kp));
+    }
+    HY_TRY(hy_new(s, &s->part, part));
+    return hy_new(s, &s->attn_cnt, ncnt);
+}
+
+int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out) {
+    const sli_stack_config& c = *cfg;
+    SLI_CHECK(c.vocab > 0 && c.width > 0 && c.n_blocks > 0 && c.blocks && c.max_len > 0 && c.batch > 0, SLI_ERR_SHAPE,
+              "stack: non-positive dimension");
+    SLI_CHECK(c.taps >= 1 && c.taps <= kCanonMaxTaps, SLI_ERR_SHAPE, "stack: taps must be 1 .. 32");
+    SLI_CHECK(c.loop_start >= 0 && c.loop_start <= c.loop_stop && c.loop_stop <= c.n_blocks && c.loop_times >= 1,
+              SLI_ERR_SHAPE, "stack: bad loop");
+    SLI_CHECK(c.w_dtype == SLI_DT_F16 || c.w_dtype == SLI_DT_F32, SLI_ERR_ARG, "stack: fp16 or fp32 weights");
+    SLI_CHECK(c.arrangement == SLI_STACK_PARALLEL || c.arrangement == SLI_STACK_SEQUENTIAL, SLI_ERR_ARG,
+              "stack: unknown arrangement");
+    SLI_CHECK(c.positions >= 0 && (c.positions == 0 || c.max_len <= c.positions), SLI_ERR_SHAPE,
+              "stack: max_len exceeds the learned positions");
+    BlockStack* s = new BlockStack();
+    *out = s;  // destroyed by the caller on failure
+    s->c = c;
+    s->stream = stream;
+    s->f16 = c.w_dtype == SLI_DT_F16;
+    s->wb = s->f16 ? 2 : 4;
+    s->D = c.width;
+    s->Dp = pad_to(c.width, 64);
+    s->V = c.vocab;
+    s->Vp = pad_to(c.vocab, 128);
+    s->T = c.max_len;
+    s->B = c.batch;
+    s->taps = std::max(c.taps, kCanonFusedTaps);
+    s->M = kHyMaxRows;
+    if (c.arrangement == SLI_STACK_SEQUENTIAL) s->seq = std::make_unique<SeqState>();
+    auto add_run = [&](int i) {
+        HyRun r;
+        r.layer = i;
+        s->runs.push_back(r);
+    };
+    if (c.runs) {
+        for (int i = 0; i < c.n_runs; ++i) {
+            SLI_CHECK(c.runs[i] >= 0 && c.runs[i] < c.n_blocks, SLI_ERR_SHAPE, "stack: a run of no block");
+            add_run(c.runs[i]);
+        }
+    } else {
+        for (int i = 0; i < c.loop_start; ++i) add_run(i);
+        for (int t = 0; t < c.loop_times; ++t)
+            for (int i = c.loop_start; i < c.loop_stop; ++i) add_run(i);
+        for (int i = c.loop_stop; i < c.n_blocks; ++i) add_run(i);
+    }
+    SLI_CHECK(!s->runs.empty(), SLI_ERR_SHAPE, "stack: no runs");
     HY_TRY(hy_alloc(s, &s->emb, s->wb * (size_t)s->V * s->D));
     HY_TRY(hy_alloc(s, &s->head, s->wb * (size_t)s->Vp * s->Dp));
     HY_TRY(hy_alloc(s, (void**)&s->fnorm, sizeof(float) * s->Dp));
     HY_TRY(hy_alloc(s, (void**)&s->fnorm_p, sizeof(float) * s->Dp));
     for (const char* n : {"embed", "head", "final.norm"}) s->want[n] = false;
+    if (c.positions > 0) {
+        HY_TRY(hy_alloc(s, &s->pos, s->wb * (size_t)c.positions * s->D));
+        s->want["pos"] = false;
+    }
     const size_t M = s->M;
     HY_TRY(hy_alloc(s, (void**)&s->rows, sizeof(RowRef) * M));
     HY_TRY(hy_alloc(s, (void**)&s->segs, sizeof(SegRef) * M));
@@ -271,60 +260,30 @@ int hy_create(const sli_stack_config* cfg, hipStream_t stream, BlockStack** out)
     HY_TRY(hy_alloc(s, &s->c1, sizeof(float) * M * s->Dp));
     HY_TRY(hy_alloc(s, &s->c2, sizeof(float) * M * s->Dp));
     HY_TRY(hy_alloc(s, &s->xl, sizeof(float) * M * s->Dp));
-    HY_TRY(hy_alloc(s, (void**)&s->q, sizeof(float) * M * nq));
-    HY_TRY(hy_alloc(s, (void**)&s->k, sizeof(float) * M * nk));
-    HY_TRY(hy_alloc(s, (void**)&s->v, sizeof(float) * M * nv));
-    HY_TRY(hy_alloc(s, (void**)&s->g, sizeof(float) * M * nv));
-    HY_TRY(hy_alloc(s, (void**)&s->o, sizeof(float) * M * no));
     HY_TRY(hy_alloc(s, (void**)&s->lg, sizeof(float) * kHyLogitRows * s->V));
-    size_t nssq = 0;
-    for (const HyLayer& l : s->layers) nssq = std::max(nssq, (size_t)l.d.heads * l.nsl);
-    HY_TRY(hy_alloc(s, (void**)&s->ssq, sizeof(float) * nssq));
-    const int Bp = s->B <= kBgMaxBatch ? s->B : pad_to(s->B, kHyTile);
-    size_t part = 0, ncnt = 0, bgp = 0, bgc = 1;
-    for (const HyLayer& l : s->layers) {
-        if (l.d.mixer == SLI_MIX_ATTENTION)
-            part = std::max(part, (size_t)Bp * l.d.heads * hy_attn_splits(s->T) * (l.hd + kAttnPartPad)),
-            ncnt = std::max(ncnt, (size_t)Bp * l.d.heads);
-        if (s->f16)
-            for (auto [np, K] : {std::make_pair(l.e_g, s->Dp), std::make_pair((int)l.d.ff, s->Dp),
-                                 std::make_pair((s->D + 1) / 2, l.Kp), std::make_pair((s->V + 1) / 2, s->Dp)})
-                for (int b = 1; b <= kBgMaxBatch; ++b) {  // (the head takes any number of wanted rows)
-                    if (np == 0) continue;
-                    const BgPlan p = bg_plan((np + 7) / 8, K, b, false, gemv_max_blocks());
-                    SLI_CHECK(p.groups > 0, SLI_ERR_SHAPE, "stack: no tiling of a batched projection fits");
-                    bgp = std::max(bgp, bg_part_bytes(p));
-                    bgc = std::max(bgc, (size_t)p.groups);
-                }
-    }
-    HY_TRY(hy_alloc(s, (void**)&s->part, sizeof(float) * part));
-    HY_TRY(hy_alloc(s, (void**)&s->attn_cnt, sizeof(unsigned) * ncnt));
-    HY_TRY(hy_alloc(s, (void**)&s->bg_ws, bgp + 256));
-    HY_TRY(hy_alloc(s, (void**)&s->bg_cnt, sizeof(unsigned) * bgc));
+    HY_TRY(hy_bg_need(s, (s->V + 1) / 2, s->Dp));
+    HY_TRY(s->seq ? seq_create(s) : par_create(s));
+    HY_TRY(hy_alloc(s, (void**)&s->bg_ws, s->bg_ws_bytes + 256));
+    HY_TRY(hy_new(s, &s->bg_cnt, s->bg_groups));
     return hy_allow_lds();
 }
 
 void hy_destroy(BlockStack* s) {
     if (!s) return;
-    for (auto* v : {&s->graphs_one, &s->graphs_rows})
-        for (auto& g : *v) {
-            if (g.second) (void)hipGraphExecDestroy(g.second);
-            if (g.first) (void)hipGraphDestroy(g.first);
-        }
+    for (auto& [key, g] : s->graphs) {
+        if (g.second) (void)hipGraphExecDestroy(g.second);
+        if (g.first) (void)hipGraphDestroy(g.first);
+    }
     for (void* p : s->allocs) (void)hipFree(p);
     delete s;
 }
 
 int hy_runs(const BlockStack* s) { return (int)s->runs.size(); }
+int hy_key_tiles(const BlockStack* s, int pos0, int n) { return seq_key_tiles(s, pos0, n); }
+int hy_key_tiles_max(const BlockStack* s) { return s->seq ? s->seq->key_tiles : 0; }
 
 // ---------------------------------------------------------------- weights
-// where a tensor's elements come from: host memory, or (host null) a generator on the device
-struct HyFill {
-    const float* host = nullptr;
-    HySrcRand rand{};
-};
-
-static int hy_place(BlockStack* s, void* dst, int ld, int col0, const std::vector<int32_t>& map, int ncols,
+int hy_place(BlockStack* s, void* dst, int ld, int col0, const std::vector<int32_t>& map, int ncols,
                     const HyFill& f) {
     const size_t n = map.size() * (size_t)ncols;
     float* tmp = nullptr;
@@ -366,7 +325,7 @@ static std::vector<int32_t> head_rows(int heads, int n, int rh, int u0) {
         }
     return map;
 }
-static std::vector<int32_t> strided_rows(int n, int first, int step) {
+std::vector<int32_t> strided_rows(int n, int first, int step) {
     std::vector<int32_t> map(n);
     for (int i = 0; i < n; ++i) map[i] = first + step * i;
     return map;
@@ -382,12 +341,17 @@ static void hy_shape(const BlockStack* s, const std::string& name, int* li, std:
         return;
     }
     if (name == "final.norm") {
-        *rows = *cols = 1;
+        *rows = 1, *cols = s->seq ? s->D : 1;
+        return;
+    }
+    if (name == "pos") {
+        *rows = s->c.positions, *cols = s->D;
         return;
     }
     const size_t dot = name.find('.');
     *li = std::atoi(name.c_str() + 1);
     *leaf = name.substr(dot + 1);
+    if (s->seq) return seq_shape(s, *li, *leaf, rows, cols);
     const sli_block_desc& d = s->layers[*li].d;
     const int kvh = d.mixer == SLI_MIX_ATTENTION ? d.kv_heads : d.heads;
     const std::string& t = *leaf;
@@ -422,8 +386,12 @@ static int hy_put(BlockStack* s, const std::string& name, const HyFill& f, int64
         rc = hy_place(s, s->emb, s->D, 0, strided_rows(s->V, 0, 1), s->D, f);
     } else if (name == "head") {
         rc = hy_place(s, s->head, s->Dp, 0, strided_rows(s->V, 0, 1), s->D, f);
+    } else if (name == "pos") {
+        rc = hy_place(s, s->pos, s->D, 0, strided_rows(s->c.positions, 0, 1), s->D, f);
     } else if (name == "final.norm") {
-        s->fgain = host[0];
+        s->fgain.assign(host, host + n);
+    } else if (s->seq) {
+        rc = seq_put(s, li, t, f);
     } else {
         HyLayer& l = s->layers[li];
         const sli_block_desc& d = l.d;
@@ -467,14 +435,16 @@ int hy_init_synthetic(BlockStack* s, uint32_t seed) {
         int64_t rows, cols;
         hy_shape(s, name, &li, &t, &rows, &cols);
         const int64_t n = rows * cols;
-        const bool canon = t == "canon1" || t == "canon2", gain = t == "norm1" || t == "norm2" || t == "final.norm";
+        const bool canon = t == "canon1" || t == "canon2";
+        const bool gain = t == "norm1" || t == "norm2" || t == "final.norm" || t == "mix.dkv.norm";
         HyFill f;
         f.rand.seed = (seed * 0x9E3779B9u) ^ (++id * 0x85EBCA6Bu);
         f.rand.amp = canon ? 0.3f : t == "embed" ? 1.0f : rows > 1 ? 1.5f / std::sqrt((float)cols) : 1.0f;
         std::vector<float> v;
         if (rows == 1 || canon) {
             const float amp = gain ? 0.1f : t == "mix.r2" ? 0.2f : f.rand.amp;
-            const float off = gain ? 1.0f : t == "mix.r2" ? 0.25f : canon ? 0.0f : 1.0f;
+            const bool bias = t.size() > 2 && t.compare(t.size() - 2, 2, ".b") == 0;
+            const float off = gain ? 1.0f : t == "mix.r2" ? 0.25f : canon || bias ? 0.0f : 1.0f;
             uint64_t x = 0x9E3779B97F4A7C15ull * (f.rand.seed + 1ull);
             for (int64_t i = 0; i < n; ++i) {
                 x ^= x >> 12, x ^= x << 25, x ^= x >> 27;
@@ -487,29 +457,32 @@ int hy_init_synthetic(BlockStack* s, uint32_t seed) {
     return SLI_OK;
 }
 
+int hy_fold_taps(BlockStack* s, const std::vector<float>& w, float gain, float* dst) {
+    const int given = s->c.taps;
+    std::vector<float> f((size_t)s->taps * s->Dp, 0.0f);
+    for (int d = 0; d < s->D; ++d)
+        for (int j = 0; j < given; ++j) {
+            const double c = (double)w[(size_t)d * given + given - 1 - j] + (j == 0 ? 1.0 : 0.0);
+            f[(size_t)j * s->Dp + d] = (float)(gain * c);
+        }
+    SLI_HIP(hipMemcpy(dst, f.data(), sizeof(float) * f.size(), hipMemcpyHostToDevice));
+    return SLI_OK;
+}
+
 int hy_prepare(BlockStack* s) {
     if (!s->dirty) return SLI_OK;
     for (auto& kv : s->want) SLI_CHECK(kv.second, SLI_ERR_STATE, "tensor '" + kv.first + "' was not loaded");
     SLI_HIP(hipStreamSynchronize(s->stream));
-    const int given = s->c.taps, Dp = s->Dp;
+    const int Dp = s->Dp;
+    if (s->seq) HY_TRY(seq_prepare(s));
     for (HyLayer& l : s->layers) {
-        auto fold = [&](const std::vector<float>& w, float gain, float* dst) -> int {
-            std::vector<float> f((size_t)s->taps * Dp, 0.0f);
-            for (int d = 0; d < s->D; ++d)
-                for (int j = 0; j < given; ++j) {
-                    const double c = (double)w[(size_t)d * given + given - 1 - j] + (j == 0 ? 1.0 : 0.0);
-                    f[(size_t)j * Dp + d] = (float)(gain * c);
-                }
-            SLI_HIP(hipMemcpy(dst, f.data(), sizeof(float) * f.size(), hipMemcpyHostToDevice));
-            return SLI_OK;
-        };
-        HY_TRY(fold(l.c1, l.n1, l.f1));
-        if (l.d.ff > 0) HY_TRY(fold(l.c2, l.n2, l.f2));
+        HY_TRY(hy_fold_taps(s, l.c1, l.n1, l.f1));
+        if (l.d.ff > 0) HY_TRY(hy_fold_taps(s, l.c2, l.n2, l.f2));
     }
     std::vector<float> g(Dp, 0.0f);
-    std::fill(g.begin(), g.begin() + s->D, s->fgain);
+    for (int d = 0; d < s->D; ++d) g[d] = s->fgain[s->fgain.size() == 1 ? 0 : d];
     SLI_HIP(hipMemcpy(s->fnorm, g.data(), sizeof(float) * Dp, hipMemcpyHostToDevice));
-    std::fill(g.begin(), g.begin() + s->D, (float)(s->fgain * std::sqrt((double)s->D / Dp)));
+    for (int d = 0; d < s->D; ++d) g[d] = (float)(g[d] * std::sqrt((double)s->D / Dp));
     SLI_HIP(hipMemcpy(s->fnorm_p, g.data(), sizeof(float) * Dp, hipMemcpyHostToDevice));
     s->dirty = false;
     return SLI_OK;
@@ -517,91 +490,12 @@ int hy_prepare(BlockStack* s) {
 
 // ---------------------------------------------------------------- the forward pass over rows
 template <typename WT>
-struct HyRec {
+struct HyRec : HyProj<WT> {
     using KT = WT;  // fp16 weights with an fp16 cache, fp32 with fp32
-    BlockStack* s;
-    int M;      // rows of the launches
-    bool one;   // one row per sequence (decode)
-    int msegs;  // portions at most
-    hipStream_t st() const { return s->stream; }
-
-    // How a projection over M rows runs: the batch-1 GEMV, the batched MFMA projection (fp16, 2 .. 8 rows; one row past
-    // the GEMV's LDS stage), the prompt GEMM (fp16, more rows), or the plain kernel (fp32, more rows or wider).
-    enum Path { GV, BG, PG, RG };
-    static constexpr bool F16 = std::is_same<WT, __half>::value;
-    static Path path(int M, int K) {
-        if (M == 1 && K <= kGemvMaxCols) return GV;
-        if (!F16) return RG;
-        return M <= kBgMaxBatch ? BG : PG;
-    }
-    // rows of the launches for n rows
-    static int rows_for(int n) { return F16 && n > kBgMaxBatch ? pad_to(n, kHyTile) : n; }
-
+    using P = HyProj<WT>;
+    using P::F16, P::GV, P::s, P::M, P::one, P::msegs, P::key_tiles, P::st, P::path, P::rows_for, P::project, P::pgemm;
     template <class Epi>
-    int project(const void* W, const void* X, int K, int npairs, int u0, const Epi& e) const {
-        const WT* w = (const WT*)W + (size_t)2 * u0 * K;
-        const Path p = path(M, K);
-        if (p == GV) {
-            GemvIn in{(const float*)X, nullptr, 0.0f, K};
-            SLI_HIP((launch_gemv_u<WT, 2, 4, true>(w, in, GvPair<Epi>{e, npairs, u0}, npairs, st())));
-            return SLI_OK;
-        }
-        if constexpr (F16) {
-            if (p == BG) {
-                BgIn in{};
-                in.x = (const float*)X;
-                in.K = K;
-                in.B = M;
-                in.ws = s->bg_ws;
-                in.counters = s->bg_cnt;
-                const BgPlan pl = bg_plan((npairs + 7) / 8, K, M, false, gemv_max_blocks());
-                SLI_HIP((launch_bgemm(w, in, BgPair<Epi>{e, npairs, u0}, pl, st())));
-                return SLI_OK;
-            }
-            if (p == PG) return pgemm(w, (const __half*)X, nullptr, 0, K, npairs, u0, e);
-        }
-        SLI_HIP((launch_rows_gemm<WT, Epi>(w, (const float*)X, K, npairs, u0, M, e, st())));
-        return SLI_OK;
-    }
-    // pairs [0, split) read X, pairs [split, npairs) X2 (split: a multiple of kHySection; X2 null: one input)
-    template <class Epi>
-    int pgemm(const WT* w, const __half* X, const __half* X2, int split, int K, int npairs, int u0, const Epi& e) const {
-        if constexpr (F16) {
-            PgIn<__half> in{w, X, nullptr, pad_to(2 * npairs, 16), K, M};
-            if (X2) in.Bhi2 = X2, in.row_b2 = 2 * split;
-            return pg_pick(M, in.N, [&](auto cfg) -> int {
-                SLI_HIP((launch_pgemm<PgPair<Epi>, decltype(cfg), __half>(in, PgPair<Epi>{e, npairs, u0}, nullptr, st())));
-                return SLI_OK;
-            });
-        } else {
-            return fail(SLI_ERR_ARG, "prompt GEMM: fp16 weights");
-        }
-    }
-    // Tilings (their row count divides M) by rows and output tiles, the fastest of a sweep at 4096 x 15104 and 34304 x 4096 with the weights streamed
-    // from HBM (TFLOP/s at 1024 rows 794 and 814, at 512 591 and 658, at 256 296 and 579): one 256 x 256 tile per CU
-    // where the grid fills the chip with them, smaller tiles (a full grid) where the output is narrow.
-    template <class F>
-    static int pg_pick(int M, int N, F&& f) {
-        const long long t128 = (long long)((N + 127) / 128) * (M / 128);
-        if (M % 256 == 0 && M != 512 && t128 >= 512) return f(PgCfg<256, 4, 2, 4, true, 0, 1>{});
-        if (M % 128 == 0 && M >= 512 && t128 >= 512) return f(PgCfg<128, 4, 2, 2, true, 0, 1>{});
-        if (M % 128 == 0 && t128 >= 256) return f(PgCfg<128, 2, 3, 4, true, 0, 1>{});
-        if (M % 64 == 0 && M >= 128) return f(PgCfg<64, 4, 4, 2, true, 0, 1>{});
-        if (M % 64 == 0) return f(PgCfg<64, 2, 4, 2, true, 0, 1>{});
-        return f(PgCfg<32, 2, 4, 2, true, 0, 1>{});
-    }
-    template <class Epi>
-    static int allow() {
-        if constexpr (F16) {
-            for (auto [M, N] : {std::make_pair(32, 128), {64, 128}, {128, 128}, {128, 1 << 15}, {256, 1 << 15}, {512, 1 << 15}})
-                HY_TRY(pg_pick(M, N, [&](auto cfg) -> int {
-                    SLI_HIP((pgemm_allow_lds<PgPair<Epi>, decltype(cfg), __half>()));
-                    return SLI_OK;
-                }));
-            SLI_HIP((bg_allow_lds<BgPair<Epi>, false>()));
-        }
-        return SLI_OK;
-    }
+    static int allow() { return P::template allow<Epi>(); }
     template <typename OT>
     static OT* cat(const HyLayer& l) {
         if constexpr (std::is_same<OT, float>::value)
@@ -725,9 +619,9 @@ struct HyRec {
                     const PfRowsArgs px{s->rows, l.r1, l.r2, l.sink, l.Kp, d.vdim};
                     const dim3 gr(M / 16, d.heads);
                     if (l.hd == 64)
-                        hipLaunchKernelGGL((pf_attn_mfma_kernel<64, true>), gr, dim3(256), 0, st(), pa, nullptr, px);
+                        hipLaunchKernelGGL((pf_attn_mfma_kernel<64, 1>), gr, dim3(256), 0, st(), pa, nullptr, px);
                     else
-                        hipLaunchKernelGGL((pf_attn_mfma_kernel<128, true>), gr, dim3(256), 0, st(), pa, nullptr, px);
+                        hipLaunchKernelGGL((pf_attn_mfma_kernel<128, 1>), gr, dim3(256), 0, st(), pa, nullptr, px);
                     SLI_HIP(hipGetLastError());
                     return SLI_OK;
                 }
@@ -805,8 +699,8 @@ struct HyRec {
         return project(l.wout, cat<OT>(l), l.Kp, (s->D + 1) / 2, 0, eo);
     }
     int embed() const {
-        hipLaunchKernelGGL(hy_embed_kernel<WT>, dim3(M), dim3(256), 0, st(), s->rows, (const WT*)s->emb, s->c.emb_scale,
-                           s->x, s->V, s->D, s->Dp);
+        hipLaunchKernelGGL(hy_embed_kernel<WT>, dim3(M), dim3(256), 0, st(), s->rows, (const WT*)s->emb, (const WT*)s->pos,
+                           s->c.emb_scale, s->x, s->V, s->D, s->Dp);
         SLI_HIP(hipGetLastError());
         return SLI_OK;
     }
@@ -827,9 +721,11 @@ struct HyRec {
     }
     int pass() const {
         HY_TRY(embed());
+        if (s->seq) return seq_pass(s, M, one, msegs, key_tiles);
         for (const HyRun& r : s->runs) HY_TRY(layer(r));
         return SLI_OK;
     }
+    int run(size_t r) const { return s->seq ? seq_run(s, M, one, msegs, key_tiles, r) : layer(s->runs[r]); }
     int step(const DevState* dst, int B, float* y, unsigned long long* keys, int key_ld, int* nkeys) const {
         hipLaunchKernelGGL(hy_rows_kernel, dim3(1), dim3(256), 0, st(), dst, s->rows, B, M);
         SLI_HIP(hipGetLastError());
@@ -865,21 +761,23 @@ static int hy_allow_lds() {
     return HyRec<__half>::allow_all();
 }
 
-#define HY_DISPATCH(s, M, one, msegs, CALL) \
-    ((s)->f16 ? HyRec<__half>{(s), (M), (one), (msegs)}.CALL : HyRec<float>{(s), (M), (one), (msegs)}.CALL)
+#define HY_DISPATCH(s, M, one, msegs, kt, CALL)                             \
+    ((s)->f16 ? HyRec<__half>{{(s), (M), (one), (msegs), (kt)}}.CALL \
+              : HyRec<float>{{(s), (M), (one), (msegs), (kt)}}.CALL)
 
 int hy_key_ld(const BlockStack*, int) { return std::max(1, gemv_max_blocks()); }
 
 int hy_record_step(BlockStack* s, const DevState* st, int B, float* logits, unsigned long long* keys, int key_ld,
                    int* nkeys) {
     const int M = s->f16 ? HyRec<__half>::rows_for(B) : B;
-    return HY_DISPATCH(s, M, true, M, step(st, B, logits, keys, key_ld, nkeys));
+    return HY_DISPATCH(s, M, true, M, 0, step(st, B, logits, keys, key_ld, nkeys));
 }
 
-static int hy_capture(BlockStack* s, std::pair<hipGraph_t, hipGraphExec_t>& g, int M, bool one, int msegs) {
+static int hy_capture(BlockStack* s, std::pair<hipGraph_t, hipGraphExec_t>& g, int M, bool one, int msegs,
+                      int key_tiles) {
     if (g.second) return SLI_OK;
     SLI_HIP(hipStreamBeginCapture(s->stream, hipStreamCaptureModeRelaxed));
-    const int rc = HY_DISPATCH(s, M, one, msegs, pass());
+    const int rc = HY_DISPATCH(s, M, one, msegs, key_tiles, pass());
     hipGraph_t gr = nullptr;
     const hipError_t e = hipStreamEndCapture(s->stream, &gr);
     if (rc != SLI_OK || e != hipSuccess) {
@@ -896,11 +794,18 @@ int hy_pass(BlockStack* s, const std::vector<RowRef>& rows_in, const std::vector
     const int n = (int)rows_in.size();
     SLI_CHECK(n >= 1 && n <= s->M && !segs.empty() && (int)segs.size() <= s->M, SLI_ERR_SHAPE, "pass: too many rows");
     // a decode step runs its rows as they are; a prompt pass is padded to a row count with a captured graph
-    int M = s->f16 ? HyRec<__half>::rows_for(n) : n, gi = M - 1;
+    int M = s->f16 ? HyRec<__half>::rows_for(n) : n, kt = 0;
     SLI_CHECK(!one || n <= s->B, SLI_ERR_SHAPE, "pass: more sequences than slots");
     if (!one) {
-        M = kHyTile, gi = 0;
-        while (M < n) M *= 2, ++gi;
+        M = kHyTile;
+        while (M < n) M *= 2;
+        for (const SegRef& g : segs) kt += seq_key_tiles(s, g.pos0, g.n);
+        SLI_CHECK(kt <= hy_key_tiles_max(s), SLI_ERR_SHAPE, "pass: too many expanded rows");
+        if (kt > 0) {  // (the grid of the expansion: a power of two, so that few graphs are captured)
+            int p = M / kLatTile + 1;
+            while (p < kt) p *= 2;
+            kt = std::min(p, hy_key_tiles_max(s));
+        }
     }
     std::vector<RowRef> rows(rows_in);
     rows.resize(M, RowRef{-1, 0, 0, 0});
@@ -910,25 +815,24 @@ int hy_pass(BlockStack* s, const std::vector<RowRef>& rows_in, const std::vector
     SLI_HIP(hipMemcpyAsync(s->nsegs, &ns, sizeof(ns), hipMemcpyHostToDevice, s->stream));
     const int msegs = one ? M : std::min(s->B, M / kHyTile);
     if (hidden_host) {  // eager, with a copy after every run
-        HY_TRY(HY_DISPATCH(s, M, one, msegs, embed()));
+        HY_TRY(HY_DISPATCH(s, M, one, msegs, kt, embed()));
         for (size_t r = 0; r < s->runs.size(); ++r) {
-            HY_TRY(HY_DISPATCH(s, M, one, msegs, layer(s->runs[r])));
+            HY_TRY(HY_DISPATCH(s, M, one, msegs, kt, run(r)));
             SLI_HIP(hipMemcpy2DAsync(hidden_host + r * (size_t)n * s->D, sizeof(float) * s->D, s->x, sizeof(float) * s->Dp,
                                      sizeof(float) * s->D, n, hipMemcpyDeviceToHost, s->stream));
         }
     } else {
-        auto& gs = one ? s->graphs_one : s->graphs_rows;
-        if ((int)gs.size() <= gi) gs.resize(gi + 1, {nullptr, nullptr});
+        auto& g = s->graphs[{one ? 0 : 1 + kt, M}];
         SLI_HIP(hipStreamSynchronize(s->stream));
-        HY_TRY(hy_capture(s, gs[gi], M, one, msegs));
-        SLI_HIP(hipGraphLaunch(gs[gi].second, s->stream));
+        HY_TRY(hy_capture(s, g, M, one, msegs, kt));
+        SLI_HIP(hipGraphLaunch(g.second, s->stream));
     }
     if (!want.empty()) {
         const int nw = (int)want.size();
         SLI_HIP(hipMemcpyAsync(s->widx, want.data(), sizeof(int32_t) * nw, hipMemcpyHostToDevice, s->stream));
         for (int w = 0; w < nw; w += kHyLogitRows) {
             const int n = std::min(kHyLogitRows, nw - w);
-            HY_TRY(HY_DISPATCH(s, M, one, msegs, logits(s->widx + w, n, s->lg)));
+            HY_TRY(HY_DISPATCH(s, M, one, msegs, kt, logits(s->widx + w, n, s->lg)));
             SLI_HIP(hipMemcpyAsync(logits_host + (size_t)w * s->V, s->lg, sizeof(float) * (size_t)n * s->V,
                                    hipMemcpyDeviceToHost, s->stream));
         }
@@ -952,11 +856,16 @@ __global__ void hy_fill_kernel(void* p, size_t n, int f16, uint32_t seed) {
 
 int hy_fill_context(BlockStack* s, uint32_t seed, int) {
     for (HyRun& r : s->runs) {
-        const HyLayer& l = s->layers[r.layer];
         auto fill = [&](void* p, size_t n, int f16) {
             if (p) hipLaunchKernelGGL(hy_fill_kernel, dim3(1024), dim3(256), 0, s->stream, p, n, f16, seed);
         };
         fill(r.ring, (size_t)s->B * s->taps * s->Dp, 0);
+        if (s->seq) {
+            fill(r.kc, (size_t)s->B * s->T * s->seq->layers[r.layer].Rp, s->f16);
+            SLI_HIP(hipGetLastError());
+            continue;
+        }
+        const HyLayer& l = s->layers[r.layer];
         fill(r.S, (size_t)s->B * l.d.heads * l.nsl * l.d.dim * kRetCols, 0);
         const size_t n = (size_t)s->B * l.d.kv_heads * s->T * l.hd;
         fill(r.kc, n, s->f16);
@@ -969,6 +878,10 @@ int hy_fill_context(BlockStack* s, uint32_t seed, int) {
 void hy_step_bytes(const BlockStack* s, int B, double pos_sum, double* weight_bytes, double* state_bytes) {
     double w = (double)s->V * s->D * s->wb, k = 0.0;
     for (const HyRun& r : s->runs) {
+        if (s->seq) {
+            seq_step_bytes(s, r, B, pos_sum, &w, &k);
+            continue;
+        }
         const HyLayer& l = s->layers[r.layer];
         const sli_block_desc& d = l.d;
         w += s->wb * (2.0 * (l.e_g + d.ff) * s->D + (double)s->D * (l.mixw + d.ff));

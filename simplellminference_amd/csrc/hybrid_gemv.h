@@ -19,6 +19,9 @@ struct XStageCanon {
     CanonArgs a;
     const float* f;  // this sublayer's coefficients
     bool write;      // this workgroup stores the new ring row
+    using Args = CanonArgs;
+    __device__ __forceinline__ XStageCanon(const CanonArgs& a_, bool second, bool first_block)
+        : a(a_), f(second ? a_.f2 : a_.f1), write(first_block) {}
     float4 x, r[kCanonFusedTaps], c[kCanonFusedTaps];
     int pos = 0, slot = 0;
     __device__ __forceinline__ void issue(const GemvIn& in) {
@@ -64,23 +67,24 @@ struct XStageCanon {
 };
 
 // workgroups [0, b1): pairs [0, n1) with the first sublayer's input; [b1, grid): pairs [u2, u2 + n2) with the second's
-template <typename WT, class Epi, bool SPLIT>
-__global__ void __launch_bounds__(kGemvThreads) hy_in_kernel(const WT* __restrict__ W, GemvIn in_, CanonArgs a, Epi epi,
-                                                             int n1, int u2, int n2, int b1) {
+// (Stage(args, second, first workgroup): what a range stages)
+template <typename WT, class Epi, class Stage, bool SPLIT>
+__global__ void __launch_bounds__(kGemvThreads) hy_in_kernel(const WT* __restrict__ W, GemvIn in_, typename Stage::Args a,
+                                                             Epi epi, int n1, int u2, int n2, int b1) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
-    constexpr int G = Vec16<WT>::N / 4;
     const bool second = (int)blockIdx.x >= b1;  // uniform
     GemvIn in = in_;
     in.blk0 = second ? b1 : 0;
     in.blk1 = second ? (int)gridDim.x : b1;
-    XStageCanon<G> stage{a, second ? a.f2 : a.f1, blockIdx.x == 0};
+    Stage stage(a, second, blockIdx.x == 0);
     GvPair<Epi> e{epi, second ? n2 : n1, second ? u2 : 0};
-    gemv_block<WT, 2, 4, true, GvPair<Epi>, XStageCanon<G>, 2, SPLIT, true>(W + (second ? (size_t)2 * u2 * in.cols : 0), in, e,
-                                                                           stage, smem);
+    gemv_block<WT, 2, 4, true, GvPair<Epi>, Stage, 2, SPLIT, true>(W + (second ? (size_t)2 * u2 * in.cols : 0), in, e, stage,
+                                                                   smem);
 }
 
-template <typename WT, class Epi>
-hipError_t launch_hy_in(const WT* W, const CanonArgs& a, const Epi& epi, int n1, int u2, int n2, hipStream_t s) {
+template <typename WT, template <int> class StageT = XStageCanon, class Epi, class SA>
+hipError_t launch_hy_in(const WT* W, const SA& a, const Epi& epi, int n1, int u2, int n2, hipStream_t s) {
+    using Stage = StageT<Vec16<WT>::N / 4>;
     GemvIn in{nullptr, nullptr, 0.0f, a.ld};
     constexpr int waves = kGemvThreads / 64;
     // two column parts per pair where the rows are long enough: waves then differ by half a pair
@@ -104,9 +108,9 @@ hipError_t launch_hy_in(const WT* W, const CanonArgs& a, const Epi& epi, int n1,
     const size_t res = std::max(gemv_res_floats(n1, b1, 2, cs), n2 ? gemv_res_floats(n2, b2, 2, cs) : 0);
     const size_t lds = gemv_lds_bytes(in.cols) + sizeof(float) * res;
     if (cs > 1)
-        hipLaunchKernelGGL((hy_in_kernel<WT, Epi, true>), dim3(b1 + b2), dim3(kGemvThreads), lds, s, W, in, a, epi, n1, u2, n2, b1);
+        hipLaunchKernelGGL((hy_in_kernel<WT, Epi, Stage, true>), dim3(b1 + b2), dim3(kGemvThreads), lds, s, W, in, a, epi, n1, u2, n2, b1);
     else
-        hipLaunchKernelGGL((hy_in_kernel<WT, Epi, false>), dim3(b1 + b2), dim3(kGemvThreads), lds, s, W, in, a, epi, n1, u2, n2, b1);
+        hipLaunchKernelGGL((hy_in_kernel<WT, Epi, Stage, false>), dim3(b1 + b2), dim3(kGemvThreads), lds, s, W, in, a, epi, n1, u2, n2, b1);
     return hipGetLastError();
 }
 

@@ -18,20 +18,23 @@ namespace sli {
 // ---------------------------------------------------------------- embedding
 // rows of a decode step from the engine's states: one row per slot
 // (rows B .. M - 1: padding)
-__global__ void hy_rows_kernel(const DevState* st, RowRef* rows, int B, int M) {
+static __global__ void hy_rows_kernel(const DevState* st, RowRef* rows, int B, int M) {
     for (int b = threadIdx.x; b < M; b += blockDim.x)
         rows[b] = b < B ? RowRef{b, st[b].pos, st[b].token, b} : RowRef{-1, 0, 0, b};
 }
 
+// (pos: learned position rows [positions][D], nullable; the context never exceeds them)
 template <typename WT>
 __global__ void __launch_bounds__(256) hy_embed_kernel(const RowRef* __restrict__ rows, const WT* __restrict__ emb,
-                                                       float scale, float* __restrict__ x, int V, int D, int ld) {
+                                                       const WT* __restrict__ pos, float scale, float* __restrict__ x,
+                                                       int V, int D, int ld) {
     const int m = blockIdx.x;
     const RowRef r = rows[m];
     const bool ok = r.tok >= 0 && r.tok < V;
     for (int i = threadIdx.x; i < ld; i += 256)
         x[(size_t)m * ld + i] = r.slot < 0 || i >= D ? 0.0f
-                                : ok ? to_f32(emb[(size_t)r.tok * D + i]) * scale
+                                : ok ? to_f32(emb[(size_t)r.tok * D + i]) * scale +
+                                           (pos ? to_f32(pos[(size_t)r.pos * D + i]) : 0.0f)
                                      : __int_as_float(0x7FC00000);
 }
 
@@ -196,6 +199,25 @@ struct HyOut {
     }
 };
 
+// y[m][row] = sum
+struct HyStore {
+    float* y;
+    int ld, D;
+    __device__ void pair(int u, int m, float v0, float v1) const {
+        float* p = y + (size_t)m * ld + 2 * u;
+        if (2 * u < D) p[0] = v0;
+        if (2 * u + 1 < D) p[1] = v1;
+    }
+    __device__ void pair2(int u, int m, const float* a, bool) const {  // u even, ld a multiple of 4
+        if (2 * u + 3 < D) {
+            *reinterpret_cast<float4*>(y + (size_t)m * ld + 2 * u) = make_float4(a[0], a[1], a[2], a[3]);
+            return;
+        }
+        pair(u, m, a[0], a[1]);
+        pair(u + 1, m, a[2], a[3]);
+    }
+};
+
 struct HyLogits {
     float* y;  // [M][n]
     int n, M;
@@ -254,21 +276,31 @@ struct PgPair {  // prefill.h: plain 16-row tiles, 4 consecutive rows per store
 
 // ---------------------------------------------------------------- the plain projection
 // y = x W^T in fp32 for any row count: a workgroup owns 16 rows x 32 pairs, both operands through LDS 32 columns at a
-// time (K a multiple of 32). The fp32 models' prompt and batch form.
-template <typename WT, class Epi>
+// time (K a multiple of 32). The fp32 models' prompt and batch form. GR: row blocks with weights of their own (prefill.h
+// PgGroups, blocks of kRowsGemmTile rows).
+constexpr int kRowsGemmTile = 16;
+template <typename WT, class Epi, bool GR = false>
 __global__ void __launch_bounds__(256) rows_gemm_kernel(const WT* __restrict__ W, const float* __restrict__ X, int K,
-                                                        int npairs, int u0, int M, Epi epi) {
-    constexpr int BM = 16, BU = 32, BK = 32;
+                                                        int npairs, int u0, int M, Epi epi, PgGroups grp) {
+    constexpr int BM = kRowsGemmTile, BU = 32, BK = 32;
     __shared__ float xs[BM][BK + 1];
     __shared__ float ws[2 * BU][BK + 1];
     const int ub = blockIdx.x * BU, mb = blockIdx.y * BM;
+    int2 tile = make_int2(0, 0);
+    if constexpr (GR) {
+        if ((int)blockIdx.y >= *grp.ntiles) return;
+        tile = grp.tiles[blockIdx.y];
+        W += (size_t)tile.x * grp.wstride;
+    }
     const int tm = threadIdx.x >> 4, tu = threadIdx.x & 15;
     float acc[2][2] = {};
     for (int k0 = 0; k0 < K; k0 += BK) {
         __syncthreads();
         for (int i = threadIdx.x; i < BM * BK; i += 256) {
             const int r = i / BK, c = i % BK;
-            xs[r][c] = mb + r < M ? X[(size_t)(mb + r) * K + k0 + c] : 0.0f;
+            int m = mb + r;
+            if constexpr (GR) m = grp.rowmap ? grp.rowmap[m] : tile.y + r;
+            xs[r][c] = GR || m < M ? X[(size_t)m * K + k0 + c] : 0.0f;
         }
         for (int i = threadIdx.x; i < 2 * BU * BK; i += 256) {
             const int r = i / BK, c = i % BK;
@@ -283,7 +315,7 @@ __global__ void __launch_bounds__(256) rows_gemm_kernel(const WT* __restrict__ W
                 for (int e = 0; e < 2; ++e) acc[p][e] = fmaf(x, ws[2 * (tu + 16 * p) + e][k], acc[p][e]);
         }
     }
-    if (mb + tm >= M) return;
+    if (!GR && mb + tm >= M) return;
 #pragma unroll
     for (int p = 0; p < 2; ++p)
         if (ub + tu + 16 * p < npairs) epi.pair(u0 + ub + tu + 16 * p, mb + tm, acc[p][0], acc[p][1]);
@@ -292,12 +324,19 @@ __global__ void __launch_bounds__(256) rows_gemm_kernel(const WT* __restrict__ W
 template <typename WT, class Epi>
 hipError_t launch_rows_gemm(const WT* W, const float* X, int K, int npairs, int u0, int M, const Epi& e, hipStream_t s) {
     hipLaunchKernelGGL((rows_gemm_kernel<WT, Epi>), dim3((npairs + 31) / 32, (M + 15) / 16), dim3(256), 0, s, W, X, K,
-                       npairs, u0, M, e);
+                       npairs, u0, M, e, PgGroups{});
+    return hipGetLastError();
+}
+template <typename WT, class Epi>
+hipError_t launch_rows_gemm_grouped(const WT* W, const float* X, int K, int npairs, const PgGroups& g, int maxtiles,
+                                    const Epi& e, hipStream_t s) {
+    hipLaunchKernelGGL((rows_gemm_kernel<WT, Epi, true>), dim3((npairs + 31) / 32, maxtiles), dim3(256), 0, s, W, X, K,
+                       npairs, 0, maxtiles * kRowsGemmTile, e, g);
     return hipGetLastError();
 }
 
 // first-maximum keys of whole logits rows: keys[b] over logits [B][n]
-__global__ void __launch_bounds__(256) hy_keys_kernel(const float* __restrict__ logits, int n,
+static __global__ void __launch_bounds__(256) hy_keys_kernel(const float* __restrict__ logits, int n,
                                                       unsigned long long* keys, int key_ld) {
     __shared__ unsigned long long red[4];
     const float* y = logits + (size_t)blockIdx.x * n;
@@ -320,15 +359,6 @@ __global__ void __launch_bounds__(256) hy_keys_kernel(const float* __restrict__ 
 struct HySrcBuf {
     const float* p;
     __device__ float operator()(size_t i) const { return p[i]; }
-};
-struct HySrcRand {  // uniform in (-amp, amp) by element index
-    uint32_t seed;
-    float amp;
-    __device__ float operator()(size_t i) const {
-        uint32_t h = (uint32_t)i * 2654435761u ^ (uint32_t)(i >> 32) * 0x9E3779B9u ^ seed;
-        h ^= h >> 16, h *= 0x7feb352du, h ^= h >> 15, h *= 0x846ca68bu, h ^= h >> 16;
-        return amp * ((float)(h >> 8) * (1.0f / 8388608.0f) - 1.0f);
-    }
 };
 template <typename WT, class Src>
 __global__ void __launch_bounds__(256) hy_place_kernel(WT* __restrict__ dst, int ld, int col0,

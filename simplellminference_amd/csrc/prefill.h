@@ -130,6 +130,16 @@ __device__ __forceinline__ void pf_wait_vm() {
     asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory");
 }
 
+// Grouped form (PgCfg::GR): row block pb of BM output rows multiplies its own weight matrix. tiles[pb] = {weight group,
+// first input row}; input row i of the block is rowmap[pb * BM + i] where a row map is given, else tiles[pb].y + i.
+// Blocks from *ntiles on (a device count; the grid is sized for the most there can be) return at once.
+struct PgGroups {
+    const int2* tiles = nullptr;
+    const int32_t* ntiles = nullptr;
+    const int32_t* rowmap = nullptr;
+    size_t wstride = 0;  // elements between two groups' weights
+};
+
 template <typename WT>
 struct PgIn {
     const WT* W;        // [N][K] fp16 or int8 (row-major, PyTorch [out][in]; int8 row scales in the epilogue)
@@ -139,6 +149,7 @@ struct PgIn {
     // weight rows from row_b2 on (a multiple of the tiling's BN) read their activations from Bhi2 (one image only)
     const __half* Bhi2 = nullptr;
     int row_b2 = 0x7fffffff;
+    PgGroups grp;
 };
 
 // Tiling: a workgroup of 2 WR waves owns BN = 32 WR weight rows x BM chunk rows; wave w holds the 2 x BM/32
@@ -158,9 +169,12 @@ struct PgIn {
 // the activation (B) images a 2-stage ring (one ahead): the A bytes come from HBM (read once per chunk), the B bytes
 // from L2, so only A needs the deep prefetch, and B, the larger image, does not pay for it in LDS.
 // NB_: activation images per position: 2 (fp16 hi + lo, two MFMAs per product) or 1 (fp16 activations; PIPE only).
-template <int BM_, int WR_, int S_, int AT_ = 2, bool PIPE_ = false, int SA_ = 0, int NB_ = 2>
+// GR_: row blocks with weights of their own (PgGroups; one image).
+template <int BM_, int WR_, int S_, int AT_ = 2, bool PIPE_ = false, int SA_ = 0, int NB_ = 2, bool GR_ = false>
 struct PgCfg {
     static_assert(NB_ == 2 || (NB_ == 1 && PIPE_), "activation images");
+    static_assert(!GR_ || NB_ == 1, "grouped: one image");
+    static constexpr bool GR = GR_;
     static constexpr int BM = BM_, WR = WR_, S = S_, AT = AT_, SA = SA_, NB = NB_;
     static constexpr bool PIPE = PIPE_;
 };
@@ -244,6 +258,12 @@ __global__ void __launch_bounds__(128 * Cfg::WR) pgemm_kernel(PgIn<WT> in, Epi e
     const int rb = (slot / PB) * 8 + xcd, pb = slot - (slot / PB) * PB;
     const int nrb = (in.N + Geo::BN - 1) / Geo::BN;
     if (rb >= nrb) return;  // (uniform) padding of the grid to a multiple of 8 row blocks
+    int2 tile = make_int2(0, 0);
+    if constexpr (Cfg::GR) {
+        if (pb >= *in.grp.ntiles) return;
+        tile = in.grp.tiles[pb];
+        in.W += (size_t)tile.x * in.grp.wstride;
+    }
     // stages: K is a multiple of 64, so with int8 weights (KS 128) the last stage may be a half stage. Its DMA
     // pieces past the row's end reload the stage's first half instead (in bounds; never read), and only its
     // first KBS / 2 k-blocks are multiplied.
@@ -279,7 +299,8 @@ __global__ void __launch_bounds__(128 * Cfg::WR) pgemm_kernel(PgIn<WT> in, Epi e
             const int r = (o2 % Geo::B_IMG) / Geo::B_ROW + lane / cpr;
             const int c = (lane % cpr) ^ pg_swz(r, Geo::B_ROW);
             const __half* B = Geo::NB == 2 ? ((u & 1) ? in.Blo : in.Bhi) : rb * Geo::BN >= in.row_b2 ? in.Bhi2 : in.Bhi;
-            const int m = pb * BM + pt * 16 + r;
+            int m = pb * BM + pt * 16 + r;
+            if constexpr (Cfg::GR) m = in.grp.rowmap ? in.grp.rowmap[m] : tile.y + pt * 16 + r;
             src[j] = reinterpret_cast<const char*>(B) + (size_t)m * in.K * 2 + c * 16;
             adv[j] = Geo::B_ROW;
             back[j] = c >= cpr / 2 ? Geo::B_ROW / 2 : 0;
@@ -713,12 +734,17 @@ __device__ __forceinline__ uint2 pa_tr_read(unsigned lds_addr) {
 // ROWS: the rows are packed portions of several sequences (step_state.h RowRef; a 16-row group belongs to one portion,
 // its valid rows first), with a distance bias and a sink per head (attn_rows.h) and one fp16 output [M][ldo] of vdim
 // dims per head; the caches hold one [hkv][T][HD] block per sequence slot.
+// ROWS 2: no bias and no sink; a query sees the last `window` positions up to its own, position t's K and V are row
+// t + koff[row / 32] of one [hkv][T][HD] block (latent.h expands them), and the output is multiplied by gate [M][hq vdim].
 struct PfRowsArgs {
     const RowRef* rows = nullptr;
     const float *r1 = nullptr, *r2 = nullptr, *sink = nullptr;  // [hq]
     int ldo = 0, vdim = 0;
+    int window = 0;
+    const int32_t* koff = nullptr;
+    const float* gate = nullptr;
 };
-template <int HD, bool ROWS = false>
+template <int HD, int ROWS = 0>
 __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a, const PfState* __restrict__ ps,
                                                            PfRowsArgs x) {
     using G = PaGeo<HD>;
@@ -730,6 +756,7 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
     const int h = blockIdx.y, kvh = h / (a.hq / a.hkv);
     const int mq = blockIdx.x * 16 + i16;  // this lane's query (chunk row)
     int pos, last, slot = 0;  // last: the group's last query position
+    int kmin = 0, koff = 0, tile0 = 0;
     bool live = true;
     if constexpr (ROWS) {
         const RowRef r0 = x.rows[blockIdx.x * 16];
@@ -738,13 +765,19 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
         live = x.rows[mq].slot >= 0;
         pos = r0.pos + i16;
         last = r0.pos + (int)__popcll(__ballot(live)) / 4 - 1;  // (a row is the query of 4 lanes)
+        if constexpr (ROWS == 2) {
+            slot = 0;
+            kmin = max(0, r0.pos - x.window + 1);  // the first key any row of the group sees
+            koff = x.koff[blockIdx.x >> 1];
+            tile0 = kmin / 32;
+        }
     } else {
         pos = ps->p0 + mq;
         last = min(ps->p0 + (int)blockIdx.x * 16 + 15, a.T - 1);
     }
     const int kmax = ROWS ? last : a.T - 1;  // cache rows past it are read as this one (their scores are masked)
     float bias1 = 0.0f, bias2 = 0.0f;
-    if constexpr (ROWS) {
+    if constexpr (ROWS == 1) {
         bias1 = x.r1[h];
         bias2 = x.r2[h];
     }
@@ -772,7 +805,7 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
     const unsigned vbase = kbase + G::IMG;
     const __half* kc = a.kc + ((size_t)slot * a.hkv + kvh) * a.T * HD;
     const __half* vc = a.vc + ((size_t)slot * a.hkv + kvh) * a.T * HD;
-    for (int tt = wave; tt < ntiles; tt += 4) {
+    for (int tt = tile0 + wave; tt < ntiles; tt += 4) {
         const int t0 = tt * 32;
         // K pieces 0 .. P/2-1, V pieces P/2 .. P-1; lane i of a piece: row (piece rows) + i / CPR, physical
         // chunk i % CPR <- logical chunk (i % CPR) ^ swizzle(row)
@@ -782,7 +815,8 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
             const int jj = isv ? j - G::PIECES / 2 : j;
             const int r = jj * (1024 / G::ROWB) + lane / G::CPR;
             const int c = (lane % G::CPR) ^ (isv ? pa_swz_v(r, G::ROWB) : pa_swz_k(r, G::ROWB));
-            const __half* src = (isv ? vc : kc) + (size_t)min(t0 + r, kmax) * HD + c * 8;
+            const int kr = ROWS == 2 ? max(min(t0 + r, kmax), kmin) + koff : min(t0 + r, kmax);
+            const __half* src = (isv ? vc : kc) + (size_t)kr * HD + c * 8;
             pf_dma(src, (isv ? vbase : kbase) + (unsigned)(jj * 1024));
         }
         pf_wait_vm<0>();
@@ -809,8 +843,9 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
             for (int r = 0; r < 4; ++r) {
                 const int key = t0 + kt * 16 + 4 * g + r;
                 float sc = sacc[kt][r] * a.scale;
-                if constexpr (ROWS) sc -= bias1 * __logf(1.0f + bias2 * (float)(pos - key));
-                const float v = key <= pos ? sc : -INFINITY;
+                if constexpr (ROWS == 1) sc -= bias1 * __logf(1.0f + bias2 * (float)(pos - key));
+                const bool see = key <= pos && (ROWS != 2 || key > pos - x.window);
+                const float v = see ? sc : -INFINITY;
                 sv[kt * 4 + r] = v;
                 cmax = fmaxf(cmax, v);
             }
@@ -886,7 +921,7 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
         M = fmaxf(M, m4[w]);
     }
     float L = 0.0f;
-    if constexpr (ROWS) {
+    if constexpr (ROWS == 1) {
         M = fmaxf(M, x.sink[h]);
         L = expf(x.sink[h] - M);
     }
@@ -905,6 +940,12 @@ __global__ void __launch_bounds__(256) pf_attn_mfma_kernel(PfAttnArgs<__half> a,
             const int d0 = t * 16 + 4 * g;
             __half* dst = a.ohi + (size_t)mq * x.ldo + (size_t)h * x.vdim + d0;
             if (!live) continue;
+            if constexpr (ROWS == 2) {
+                const float* gt = x.gate + ((size_t)mq * a.hq + h) * x.vdim + d0;
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    if (d0 + r < x.vdim) acc[r] *= gt[r];
+            }
             if (x.vdim % 4 == 0 && d0 < x.vdim) {
                 const __half hv[4] = {__float2half_rn(acc[0] * inv), __float2half_rn(acc[1] * inv),
                                       __float2half_rn(acc[2] * inv), __float2half_rn(acc[3] * inv)};

@@ -11,7 +11,7 @@ from typing import Callable
 
 from .checkpoint import read_config
 from .model import LlamaModel, LlamaModelConfig
-from .stack import Rugudra
+from .stack import Bokulix, Rugudra
 
 _REGISTRY: dict[str, Callable] = {}
 
@@ -39,6 +39,11 @@ def _llama(cfg: dict, folder: str, dtype: str, max_length: int, batch: int, devi
 @register("Rugudra")
 def _rugudra(cfg: dict, folder: str, dtype: str, max_length: int, batch: int, device: int):
     return Rugudra.from_config(cfg, max_length, model_path=folder, dtype=dtype, batch=batch, device=device)
+
+
+@register("Bokulix")
+def _bokulix(cfg: dict, folder: str, dtype: str, max_length: int, batch: int, device: int):
+    return Bokulix.from_config(cfg, max_length, model_path=folder, dtype=dtype, batch=batch, device=device)
 
 
 def load_model(folder: str, dtype: str = "bfloat16", max_length: int = 1024, batch: int = 1, device: int = 0):

@@ -1,11 +1,13 @@
 """Block-stack models (include/sli.h ``sli_stack_config``): decoders of parallel blocks with attention and retention
-mixers, behind the same engine handle, decode loop and greedy sampling as ``LlamaModel``.
+mixers, or of sequential sublayers with latent attention and mixtures of experts, behind the same engine handle, decode
+loop and greedy sampling as ``LlamaModel``.
 
-``StackModel`` takes any ``StackConfig``; ``Rugudra`` reads one design's ``config.json`` into it."""
+``StackModel`` takes any ``StackSpec``; ``Rugudra`` and ``Bokulix`` read one design's ``config.json`` into it."""
 from __future__ import annotations
 
 import ctypes
 import os
+import re
 from dataclasses import dataclass, field
 
 import numpy as np
@@ -17,13 +19,16 @@ from .model import LlamaModel
 
 # storage per --dtype: bfloat16 checkpoints are served with fp16 weights and cache (every bfloat16 value of magnitude
 # 2^-14 .. 65504 is an fp16 value), float32 in fp32 throughout
+MIXERS = ("attention", "retention", "latent")  # sli_mixer_kind
+ARRANGEMENTS = ("parallel", "sequential")  # sli_stack_arrangement
+
 DTYPES = {"bfloat16": DT_F16, "bf16": DT_F16, "float16": DT_F16, "f16": DT_F16, "fp16": DT_F16,
           "float32": DT_F32, "f32": DT_F32, "fp32": DT_F32}
 
 
 @dataclass(frozen=True)
 class BlockSpec:
-    mixer: str  # "attention" | "retention"
+    mixer: str  # of MIXERS
     heads: int
     dim: int
     vdim: int
@@ -32,8 +37,12 @@ class BlockSpec:
     decay: tuple[float, ...] = ()
     rot_dims: int = 0
     rot_base: float = 10000.0
-    ff: int = 0
+    ff: int = 0  # rows of the feed-forward (of each expert)
     ff_limit: float = 0.0
+    kv_rank: int = 0  # latent attention
+    window: int = 0  # latent attention: positions a query sees, itself included (0: all)
+    experts: int = 0  # 0: a dense feed-forward
+    top: int = 0
 
 
 @dataclass(frozen=True)
@@ -48,12 +57,32 @@ class StackSpec:
     residual_mult: float = 1.0
     max_length: int = 1024
     extra: dict = field(default_factory=dict, compare=False)
+    arrangement: str = "parallel"
+    positions: int = 0  # rows of the learned position table (0: none)
+    runs: tuple[int, ...] = ()  # block of every run (empty: by `loop`)
+    layer_names: tuple[int, ...] = ()  # block i's tensors are l<layer_names[i]>.* in the file (empty: l<i>.*)
 
     @property
     def order(self) -> list[int]:
         """Block index of every run of a forward pass."""
+        if self.runs:
+            return list(self.runs)
         a, b, n = self.loop
         return list(range(a)) + list(range(a, b)) * n + list(range(b, len(self.blocks)))
+
+    def tensor_names(self, names) -> list[tuple[str, str]]:
+        """(name in the file, name in the model) of the tensors to place. Left out: what a block without a feed-forward
+        may still name of its second sublayer."""
+        block_of = {n: i for i, n in enumerate(self.layer_names or range(len(self.blocks)))}
+        out = []
+        for name in names:
+            m = re.fullmatch(r"l(\d+)\.(.+)", name)
+            i = block_of.get(int(m[1])) if m else None
+            if i is None:
+                out.append((name, name if not m else f"l{len(self.blocks)}.{m[2]}"))  # (no block's: refused by the model)
+            elif self.blocks[i].ff or m[2] not in ("norm2", "canon2", "rg2", "rg2.b"):
+                out.append((name, f"l{i}.{m[2]}"))
+        return out
 
 
 class StackModel(LlamaModel):
@@ -80,19 +109,25 @@ class StackModel(LlamaModel):
         blocks = (BlockDesc * len(s.blocks))()
         decay: list[float] = []
         for d, b in zip(blocks, s.blocks):
-            if b.mixer not in ("attention", "retention"):
+            if b.mixer not in MIXERS:
                 raise ValueError(f"unknown mixer {b.mixer!r}")
-            d.mixer = 0 if b.mixer == "attention" else 1
+            d.mixer = MIXERS.index(b.mixer)
             d.heads, d.kv_heads, d.dim, d.vdim = b.heads, b.kv_heads, b.dim, b.vdim
             d.scale, d.rot_dims, d.rot_base = b.scale, b.rot_dims, b.rot_base
             d.ff, d.ff_limit = b.ff, b.ff_limit
+            d.kv_rank, d.window, d.experts, d.top = b.kv_rank, b.window, b.experts, b.top
             if d.mixer == 1:
                 if len(b.decay) != b.heads:
                     raise ValueError("retention: one decay per head")
                 decay += list(b.decay)
         dec = np.ascontiguousarray(decay or [0.0], np.float32)
+        if s.arrangement not in ARRANGEMENTS:
+            raise ValueError(f"unknown arrangement {s.arrangement!r}")
+        runs = np.ascontiguousarray(s.runs, np.int32)
         c = _CStackConfig(s.vocab_size, s.width, len(s.blocks), *s.loop, s.taps, s.eps, s.emb_scale, s.residual_mult,
-                          blocks, dec.ctypes.data_as(_lib.P_f), self.w_dtype, s.max_length, self.batch, self.device)
+                          blocks, dec.ctypes.data_as(_lib.P_f), self.w_dtype, s.max_length, self.batch, self.device,
+                          ARRANGEMENTS.index(s.arrangement), s.positions,
+                          runs.ctypes.data_as(_lib.P_i32) if runs.size else None, runs.size)
         h = ctypes.c_void_p()
         call("sli_stack_create", ctypes.byref(c), ctypes.byref(h))
         self._h = h
@@ -101,10 +136,8 @@ class StackModel(LlamaModel):
     def _load_weights(self) -> "StackModel":
         if self.model_path:
             st = SafeTensors(os.path.join(self.model_path, "model.safetensors"))
-            unused = {f"l{i}.{n}" for i, b in enumerate(self.spec.blocks) if not b.ff for n in ("norm2", "canon2")}
-            for name in st.names():  # (a block without a feed-forward may still name its second sublayer's norm and taps)
-                if name not in unused:
-                    self.set_tensor(name, st.get(name))
+            for name, placed in self.spec.tensor_names(st.names()):
+                self.set_tensor(placed, st.get(name))
         elif self.seed is not None:
             call("sli_model_init_synthetic", self._h, self.seed)
         return self
@@ -189,3 +222,43 @@ class Rugudra(StackModel):
     @classmethod
     def from_config(cls, cfg: dict, max_length: int, **kw) -> "Rugudra":
         return cls(rugudra_spec(cfg, max_length), **kw)
+
+
+def bokulix_spec(cfg: dict, max_length: int) -> StackSpec:
+    """A ``config.json`` of architecture "Bokulix" as a StackSpec. A layer with ``weights_of`` is another run of that
+    layer's block."""
+    blocks, names, runs, block_of = [], [], [], {}
+    for i, e in enumerate(cfg["layers"]):
+        if e.get("weights_of") is not None:
+            continue
+        if e["type"] != "latent_attention":
+            raise ValueError(f"unknown layer type {e['type']!r}")
+        m, f = e["mixer"], e.get("mlp")
+        if f is not None and f["kind"] != "moe":
+            raise ValueError(f"unknown feed-forward kind {f['kind']!r}")
+        ff = {"ff": f["expert"]["ff"], "experts": f["router"]["experts"], "top": f["router"]["top"]} if f is not None else {}
+        block_of[i] = len(blocks)
+        names.append(i)
+        blocks.append(BlockSpec("latent", m["heads"], m["dim"], m["vdim"], scale=m["scale"], kv_rank=m["kv_rank"],
+                                window=(m.get("mask") or {}).get("size", 0), **ff))
+    for i, e in enumerate(cfg["layers"]):
+        seen = {i}
+        while cfg["layers"][i].get("weights_of") is not None:
+            i = cfg["layers"][i]["weights_of"]
+            if i in seen or not 0 <= i < len(cfg["layers"]):
+                raise ValueError("weights_of names no layer with weights")
+            seen.add(i)
+        runs.append(block_of[i])
+    n = cfg["max_positions"]
+    return StackSpec(cfg["vocab"], cfg["width"], tuple(blocks), taps=cfg["canon"]["taps"], eps=cfg["norm"]["eps"],
+                     max_length=min(max_length, n), arrangement="sequential", positions=n, runs=tuple(runs),
+                     layer_names=tuple(names))
+
+
+class Bokulix(StackModel):
+    """Sequential sublayers, each gated and normed on its output: windowed latent attention behind an input convolution,
+    and a mixture of experts; learned positions, layers that share their weights."""
+
+    @classmethod
+    def from_config(cls, cfg: dict, max_length: int, **kw) -> "Bokulix":
+        return cls(bokulix_spec(cfg, max_length), **kw)

@@ -71,7 +71,7 @@ def test_config_to_spec():
 
 def test_registry_names_and_unknown(tmp_path):
     from simplellminference_amd.registry import architectures, load_model
-    assert architectures() == ["Llama", "Rugudra"]
+    assert architectures() == ["Bokulix", "Llama", "Rugudra"]
     (tmp_path / "config.json").write_text('{"architecture": "Nothing"}')
     with pytest.raises(ValueError, match="unknown architecture"):
         load_model(str(tmp_path))
