@@ -134,21 +134,30 @@ def shapes(c):
 
 def random_tensors(c, seed):
     """Random weights on which every mechanism shows: scores of a few units, gates on both sides of one half, norm gains
-    away from 1, router biases that decide some choices. fp16-exact values, so both precisions hold the same model."""
+    away from 1. fp16-exact values, so both precisions hold the same model. The routers read the first quarter of the
+    channels, which no sublayer adds to (norm gains 0, no position rows): the choice of experts follows from the token,
+    and no rounding of the residual stream turns a close call into another expert."""
     r = np.random.default_rng(seed)
-    t = {}
+    t, own = {}, max(1, c["width"] // 4)
     for name, s in shapes(c).items():
         leaf = name.split(".")[-1]
         if "norm" in name:
             v = 0.6 + 0.8 * r.random(s)
+            if leaf in ("norm1", "norm2"):
+                v[:own] = 0.0
         elif leaf == "canon1":
             v = 0.35 * r.standard_normal(s)
         elif leaf in ("embed", "pos"):
             v = (1.0 if leaf == "embed" else 0.5) * r.standard_normal(s)
+            if leaf == "pos":
+                v[:, :own] = 0.0
+        elif leaf == "router":
+            v = np.zeros(s)
+            v[:, :own] = 1.5 * r.standard_normal((s[0], own)) / np.sqrt(own)
         elif len(s) == 1:
             v = 0.7 * r.standard_normal(s)
         else:
-            gain = {"q": 1.5, "uk": 1.5, "gate": 1.2, "up": 1.2, "router": 1.5, "head": 1.0}.get(leaf, 0.9)
+            gain = {"q": 1.5, "uk": 1.5, "gate": 1.2, "up": 1.2, "head": 1.0}.get(leaf, 0.9)
             v = gain * r.standard_normal(s) / np.sqrt(s[-1])
         t[name] = np.asarray(v).astype(np.float16).astype(np.float64)
     return t
