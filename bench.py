@@ -3,7 +3,8 @@
 
     python bench.py [--gpus N] [--steps K] [--warmup W]
     python bench.py --preset llama3-8b --ctx 4096 --batch 8      # BASELINE configs[4] (C4) at TP = N
-    python bench.py --design rugudra --steps 20 --warmup 5       # the block-stack design beside Llama of equal size
+    python bench.py --design bokulix --steps 20 --warmup 5       # a block-stack design beside Llama of equal size
+                                                                 # (or rugudra)
     python -m torch.distributed.run --nnodes=1 --nproc-per-node N --master-addr 127.0.0.1 \
         --master-port P bench.py --gpus N --steps K --warmup W
 
@@ -87,17 +88,18 @@ def parse():
         (p for p in (os.path.join(ROOT, "profiles", f) for f in ("r6_gemv_traffic.json", "r5_gemv_traffic.json", "r4_gemv_traffic.json",
                                                                    "r3_gemv_traffic.json"))
          if os.path.exists(p)), os.path.join(ROOT, "profiles", "r5_gemv_traffic.json")))
-    ap.add_argument("--design", default="llama", choices=["llama", "rugudra"],
-                    help="rugudra: instead of the default workload, time the block-stack design beside the Llama model "
-                         "of equal width, depth, heads, feed-forward and vocabulary (decode and prompt), one JSON line")
+    ap.add_argument("--design", default="llama", choices=["llama", "rugudra", "bokulix"],
+                    help="rugudra, bokulix: instead of the default workload, time the block-stack design beside the Llama "
+                         "model of equal width, depth, heads, feed-forward and vocabulary (decode and prompt), one JSON line")
     ap.add_argument("--design-sizes", default="1b,7b,8b", help="--design: sizes to run")
     ap.add_argument("--design-batches", default="1,8", help="--design: decode batch sizes")
     ap.add_argument("--design-prompts", default="513,1025,2000", help="--design: prompt lengths (batch 1)")
-    ap.add_argument("--design-models", default="rugudra,llama", help="--design: which of the two to time")
+    ap.add_argument("--design-models", default="", help="--design: what to time (rugudra, bokulix, llama; default: the "
+                                                        "design and llama)")
     return ap.parse_args()
 
 
-# --design: (context, Llama shape) of each size; the block stack alternates retention and attention blocks of it
+# --design: (context, Llama shape) of each size
 DESIGN_SIZES = {
     "1b": (2048, dict(vocab_size=32000, head_dim=64, hidden_size=2048, kv_hidden_size=512, intermediate_size=8192,
                       num_hidden_layers=16, num_attention_heads=32, num_key_value_heads=8)),
@@ -108,18 +110,23 @@ DESIGN_SIZES = {
 }
 
 
-def design_spec(shape: dict, ctx: int):
-    """The block stack of a Llama shape: retention with width / 256 heads of dim 128 and vdim 256, attention with the
-    Llama's heads."""
+def design_spec(design: str, shape: dict, ctx: int):
+    """A block stack of a Llama shape. rugudra: retention with width / 256 heads of dim 128 and vdim 256, alternating with
+    attention with the Llama's heads. bokulix: latent attention with the Llama's heads (rank 4 heads' width, the window half
+    the context), 8 experts of half the feed-forward, 2 per token."""
     from simplellminference_amd.stack import BlockSpec, StackSpec
-    D, ff, hd = shape["hidden_size"], shape["intermediate_size"], shape["head_dim"]
+    D, ff, hd, n = shape["hidden_size"], shape["intermediate_size"], shape["head_dim"], shape["num_hidden_layers"]
+    if design == "bokulix":
+        b = BlockSpec("latent", shape["num_attention_heads"], hd, hd, scale=hd ** -0.5, kv_rank=4 * hd, window=ctx // 2,
+                      experts=8, top=2, ff=ff // 2)
+        return StackSpec(shape["vocab_size"], D, (b,) * n, taps=4, eps=1e-6, max_length=ctx, arrangement="sequential",
+                         positions=ctx)
     rh = D // 256
     at = BlockSpec("attention", shape["num_attention_heads"], hd, hd, kv_heads=shape["num_key_value_heads"],
                    scale=hd ** -0.5, ff=ff, ff_limit=7.0)
     rt = BlockSpec("retention", rh, 128, 256, decay=tuple(1 - 2.0 ** (-5 - 4 * i / rh) for i in range(rh)), rot_dims=128,
                    rot_base=1e4, ff=ff, ff_limit=7.0)
-    return StackSpec(shape["vocab_size"], D, (rt, at) * (shape["num_hidden_layers"] // 2), taps=4, eps=1e-6,
-                     residual_mult=0.3, max_length=ctx)
+    return StackSpec(shape["vocab_size"], D, (rt, at) * (n // 2), taps=4, eps=1e-6, residual_mult=0.3, max_length=ctx)
 
 
 def design_bench(a) -> dict:
@@ -132,9 +139,9 @@ def design_bench(a) -> dict:
     for size in a.design_sizes.split(","):
         ctx, shape = DESIGN_SIZES[size]
         for B in [int(b) for b in a.design_batches.split(",")]:
-            for which in a.design_models.split(","):
-                if which == "rugudra":
-                    m = StackModel(design_spec(shape, ctx), dtype="bfloat16", batch=B, seed=1).init()
+            for which in (a.design_models or f"{a.design},llama").split(","):
+                if which != "llama":
+                    m = StackModel(design_spec(which, shape, ctx), dtype="bfloat16", batch=B, seed=1).init()
                 else:
                     m = LlamaModel(config=LlamaModelConfig(**shape, max_length=ctx, rms_norm_eps=1e-5, rope_theta=1e4), seed=1,
                                    batch=B).init()
@@ -159,14 +166,14 @@ def design_bench(a) -> dict:
                         m.prefill(ids)
                         ts.append(time.perf_counter() - t0)
                     t = statistics.median(ts)
-                    mm = w - 2.0 * shape["vocab_size"] * shape["hidden_size"]  # projection weights (fp16 bytes = flops / token)
+                    mm = w - 2.0 * shape["vocab_size"] * shape["hidden_size"]  # projection weights a token uses (fp16 bytes = flops)
                     rows.append({"size": size, "model": which, "prompt": n, "ms": round(t * 1e3, 2),
                                  "tokens_per_s": round((n - 1) / t, 1),
                                  "projection_tflops": round(mm * (n - 1) / t / 1e12, 1)})
                     progress(str(rows[-1]))
                 m.close()
-    dec = [r for r in rows if r["model"] == "rugudra" and r.get("batch") == 1]
-    return {"metric": "block-stack (Rugudra) decode tokens/s beside the Llama model of equal size, fp16, 1 MI355X",
+    dec = [r for r in rows if r["model"] == a.design and r.get("batch") == 1]
+    return {"metric": f"block-stack ({a.design.capitalize()}) decode tokens/s beside the Llama model of equal size, fp16, 1 MI355X",
             "value": dec[-1]["tokens_per_s"] if dec else None, "unit": "tokens/s", "n_gpus": 1, "steps": a.steps,
             "warmup": a.warmup, "ms_per_step": round(dec[-1]["step_us"] / 1e3, 4) if dec else None,
             "higher_is_better": True, "scaling": "strong", "vs_baseline": None, "dtype": "f16", "data": "synthetic",
