@@ -88,7 +88,10 @@ inline size_t bg_lds_bytes(int K, int splits, int tpw) {
 // staging amortised over several tiles (B*K/splits*4 bytes from L2 per workgroup, plus B*K*4 for the
 // fused RMS over the full row), the LDS image within 160 KiB. Cost in units of one 16x32 fp16 weight
 // block (1 KiB of HBM); L2 bytes priced at a quarter of HBM bytes.
-inline BgPlan bg_plan(int ntiles, int K, int B, bool norm, int cus = 256) {
+// steps (row-major weights): a wave's blocks of a tile are priced as the whole steps they take, and a split's publish and
+// merge at 3 us. At 8 rows of 4096 columns 544 tiles took 20.5 us in one split and 30.4 us in four, 257 tiles 14.8 us and
+// (five) 21.5 us.
+inline BgPlan bg_plan(int ntiles, int K, int B, bool norm, int cus = 256, bool steps = false) {
     const int nkb = K / 32;
     BgPlan best;
     double best_cost = 1e30;
@@ -105,7 +108,13 @@ inline BgPlan bg_plan(int ntiles, int K, int B, bool norm, int cus = 256) {
             const int groups = (ntiles + tpw - 1) / tpw;
             const int wgs = groups * s;
             const int rounds = (wgs + cus - 1) / cus;
-            double per_wg = (double)tpw * kbs + 0.25 * kbs * B / 8.0 + 40.0;
+            int blocks = kbs;
+            if (steps) {
+                const int bpw = (kbs + kBgWaves - 1) / kBgWaves, w = bg_seven_blocks(s, K) ? 7 : bg_step_width(tpw);
+                blocks = kBgWaves * w * ((bpw + w - 1) / w);
+            }
+            double per_wg = (double)tpw * blocks + 0.25 * kbs * B / 8.0 + 40.0;
+            if (steps && s > 1) per_wg += 80.0;
             if (norm) per_wg += 0.25 * nkb * B / 8.0;
             if (s > 1) per_wg += 20.0 + 0.5 * s * tpw;
             const double cost = rounds * per_wg;

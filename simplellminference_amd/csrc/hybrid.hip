@@ -80,7 +80,7 @@ static int hy_allow_lds();
 int hy_bg_need(BlockStack* s, int np, int K) {
     if (!s->f16 || np == 0) return SLI_OK;
     for (int b = 1; b <= kBgMaxBatch; ++b) {
-        const BgPlan p = bg_plan((np + 7) / 8, K, b, false, gemv_max_blocks());
+        const BgPlan p = bg_plan((np + 7) / 8, K, b, false, gemv_max_blocks(), true);
         SLI_CHECK(p.groups > 0, SLI_ERR_SHAPE, "stack: no tiling of a batched projection fits");
         s->bg_ws_bytes = std::max(s->bg_ws_bytes, bg_part_bytes(p));
         s->bg_groups = std::max(s->bg_groups, (size_t)p.groups);

@@ -46,7 +46,7 @@ struct HyProj {
                 in.B = M;
                 in.ws = s->bg_ws;
                 in.counters = s->bg_cnt;
-                const BgPlan pl = bg_plan((npairs + 7) / 8, K, M, false, gemv_max_blocks());
+                const BgPlan pl = bg_plan((npairs + 7) / 8, K, M, false, gemv_max_blocks(), true);
                 SLI_HIP((launch_bgemm(w, in, BgPair<Epi>{e, npairs, u0}, pl, st())));
                 return SLI_OK;
             }

@@ -448,7 +448,7 @@ struct SeqRec : HyProj<WT> {
                 SLI_HIP(hipGetLastError());
             }
             hipLaunchKernelGGL((lat_out_kernel<WT, OT>), dim3((d.vdim + kLatOutRows - 1) / kLatOutRows, d.heads, M), dim3(256),
-                               sizeof(float) * l.Rp, st(), a, cat, l.KA);
+                               lat_out_lds(l.Rp), st(), a, cat, l.KA);
             SLI_HIP(hipGetLastError());
             return SLI_OK;
         }
@@ -520,6 +520,22 @@ struct SeqRec : HyProj<WT> {
         return SLI_OK;
     }
 
+    // the choices of a pass and its expert rows' layout
+    template <int NV>
+    int route(const MoeRoute& r, int bm) const {
+        if (M <= kMoeGroupRoutes) {
+            hipLaunchKernelGGL(moe_group_kernel<NV>, dim3(1), dim3(1024), 0, st(), r, bm, q().at, q().rowmap, q().tiles,
+                               q().ntiles);
+        } else {
+            hipLaunchKernelGGL(moe_topk_kernel<NV>, dim3((M + 3) / 4), dim3(256), 0, st(), r);
+            SLI_HIP(hipGetLastError());
+            hipLaunchKernelGGL(moe_group_kernel<0>, dim3(1), dim3(1024), 0, st(), r, bm, q().at, q().rowmap, q().tiles,
+                               q().ntiles);
+        }
+        SLI_HIP(hipGetLastError());
+        return SLI_OK;
+    }
+
     // ---- any rows
     template <typename OT>
     int layer_rows(const HyRun& r) const {
@@ -553,18 +569,8 @@ struct SeqRec : HyProj<WT> {
         const void* xin = half ? (const void*)q().xh : (const void*)s->x;
         HY_TRY(project(l.wg2, xin, s->Dp, l.n2, 0, gate_epi(l)));
         const int E = d.experts, top = d.top, bm = bm_for(s, M, top, E), mt = moe_max_tiles(M * top, E, bm);
-        const dim3 tg((M + 3) / 4);
-        if (E <= 64)
-            hipLaunchKernelGGL(moe_topk_kernel<1>, tg, dim3(256), 0, st(), q().z, s->rows, M, E, top, q().sel, q().wsel);
-        else if (E <= 256)
-            hipLaunchKernelGGL(moe_topk_kernel<4>, tg, dim3(256), 0, st(), q().z, s->rows, M, E, top, q().sel, q().wsel);
-        else
-            hipLaunchKernelGGL(moe_topk_kernel<kMoeMaxExperts / 64>, tg, dim3(256), 0, st(), q().z, s->rows, M, E, top, q().sel,
-                               q().wsel);
-        SLI_HIP(hipGetLastError());
-        hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), 0, st(), q().sel, M * top, top, E, bm, q().at, q().rowmap,
-                           q().tiles, q().ntiles);
-        SLI_HIP(hipGetLastError());
+        const MoeRoute mr{q().z, s->rows, M, E, top, q().sel, q().wsel};
+        HY_TRY(E <= 64 ? route<1>(mr, bm) : E <= 256 ? route<4>(mr, bm) : route<kMoeMaxExperts / 64>(mr, bm));
         PgGroups g{};
         g.tiles = q().tiles, g.ntiles = q().ntiles, g.rowmap = q().rowmap, g.wstride = (size_t)2 * l.ffp * s->Dp;
         PgGroups gd = g;

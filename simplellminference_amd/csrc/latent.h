@@ -341,36 +341,62 @@ __global__ void __launch_bounds__(256) lat_attn_rows_kernel(LatArgs a) {
 }
 
 // The splits merged, U_v applied, the gate: out[m][h * vdim + v]. Grid (value rows / 32, H, M): a wave owns 8 value rows
-// (their first 16 bytes per lane in flight before the merge).
+// (their first 16 bytes per lane in flight before the merge). The merge: thread groups of Rp / 4 threads take every ng-th
+// split, kLatMerge loads of each in flight; lane s has split s's maximum and sum.
+constexpr int kLatMerge = 8;
+inline size_t lat_out_lds(int Rp) { return sizeof(float) * (size_t)std::max(Rp, 1024); }
 template <typename WT, typename OT>
 __global__ void __launch_bounds__(256) lat_out_kernel(LatArgs a, OT* out, int ldo) {
-    extern __shared__ __attribute__((aligned(16))) float lo_sm[];  // [Rp]
+    extern __shared__ __attribute__((aligned(16))) float lo_sm[];  // [ng][Rp]
+    __shared__ float se[kLatMaxSplits];
     constexpr int VE = Vec16<WT>::N, NR = kLatOutRows / 4;
     const int h = blockIdx.y, m = blockIdx.z, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const RowRef r = a.rows[m];
     if (r.slot < 0) return;
     const int v0 = blockIdx.x * kLatOutRows + wave * NR, nvec = a.Rp / VE;
     const WT* w = (const WT*)a.uv + (size_t)h * a.vdim * a.Rp;
+    const int ns = lat_span(r.pos, a.window, a.splits).ns, ps = a.Rp + kAttnPartPad;
+    const float* p = a.part + ((size_t)m * a.H + h) * a.splits * ps;
+    const int n4 = a.Rp / 4, ng = max(1, 256 / n4), grp = n4 > 256 ? 0 : tid / n4, c0 = tid - grp * n4;
+    float4 v[kLatMerge];
+    auto load = [&](int s0, int c) {
+#pragma unroll
+        for (int j = 0; j < kLatMerge; ++j)
+            v[j] = *reinterpret_cast<const float4*>(p + (size_t)min(s0 + j * ng, ns - 1) * ps + 4 * min(c, n4 - 1));
+    };
+    const float ms = p[(size_t)min(lane, ns - 1) * ps + a.Rp], ls = p[(size_t)min(lane, ns - 1) * ps + a.Rp + 1];
+    load(grp, c0);
     u32x4 wf[NR];
 #pragma unroll
     for (int j = 0; j < NR; ++j)
         wf[j] = load16<false>(w + (size_t)min(v0 + j, a.vdim - 1) * a.Rp + min(lane, nvec - 1) * VE);
-    const int ns = lat_span(r.pos, a.window, a.splits).ns, ps = a.Rp + kAttnPartPad;
-    const float* p = a.part + ((size_t)m * a.H + h) * a.splits * ps;
-    float M = -INFINITY, L = 0.0f;
-    for (int s = 0; s < ns; ++s) M = fmaxf(M, p[(size_t)s * ps + a.Rp]);
-    for (int s = 0; s < ns; ++s) L = fmaf(expf(p[(size_t)s * ps + a.Rp] - M), p[(size_t)s * ps + a.Rp + 1], L);
-    for (int i = tid; i < a.Rp / 4; i += 256) {
-        float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
-#pragma unroll 4
-        for (int s = 0; s < ns; ++s) {
-            const float e = expf(p[(size_t)s * ps + a.Rp] - M);
-            const float4 v = *reinterpret_cast<const float4*>(p + (size_t)s * ps + 4 * i);
-            o = fma4(v, make_float4(e, e, e, e), o);
-        }
-        reinterpret_cast<float4*>(lo_sm)[i] = make_float4(o.x / L, o.y / L, o.z / L, o.w / L);
-    }
+    const float M = wave_max(ms), e = lane < ns ? expf(ms - M) : 0.0f, L = wave_sum(e * ls);
+    if (wave == 0 && lane < kLatMaxSplits) se[lane] = e / L;  // 0 past the last split
     __syncthreads();
+    if (grp < ng)
+        for (int c = c0; c < n4; c += 256) {
+            if (c != c0) load(grp, c);
+            float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
+            for (int s0 = grp; s0 < ns; s0 += ng * kLatMerge) {
+                if (s0 != grp) load(s0, c);
+#pragma unroll
+                for (int j = 0; j < kLatMerge; ++j) {
+                    const int s = s0 + j * ng;
+                    const float es = s < kLatMaxSplits ? se[s] : 0.0f;
+                    o = fma4(v[j], make_float4(es, es, es, es), o);
+                }
+            }
+            reinterpret_cast<float4*>(lo_sm)[grp * n4 + c] = o;
+        }
+    __syncthreads();
+    if (ng > 1) {
+        for (int c = tid; c < n4; c += 256) {
+            float4 o = reinterpret_cast<const float4*>(lo_sm)[c];
+            for (int g = 1; g < ng; ++g) o = fma4(reinterpret_cast<const float4*>(lo_sm)[g * n4 + c], make_float4(1.f, 1.f, 1.f, 1.f), o);
+            reinterpret_cast<float4*>(lo_sm)[c] = o;
+        }
+        __syncthreads();
+    }
 #pragma unroll
     for (int j = 0; j < NR; ++j) {
         if (v0 + j >= a.vdim) break;  // (uniform in the wave)

@@ -1,6 +1,6 @@
 // moe.h — a mixture of experts on gfx950: each token uses the `top` experts with the largest router logits, weighted by
 // the softmax over the chosen logits; an expert is down(silu(gate h) * (up h)).
-//   * batches and prompts: moe_topk_kernel (a wave per token), moe_group_kernel sorts the (token, expert) pairs by expert
+//   * batches and prompts: moe_topk_kernel (a wave per token; a few tokens: in the next launch), moe_group_kernel sorts the (token, expert) pairs by expert
 //     into row blocks of one tile height (a stable order: the same batch gives the same blocks), then two grouped GEMMs
 //     (prefill.h PgGroups) read the token rows through the row map and write expert rows, which gated.h weights and adds;
 //   * one token: the choice runs in the prologue of the gate / up GEMV (EpiMoeUp), which streams the chosen experts'
@@ -17,6 +17,7 @@ namespace sli {
 
 constexpr int kMoeMaxExperts = 1024;
 constexpr int kMoeMaxTop = 64;
+constexpr int kMoeGroupRoutes = 16;  // rows at most whose choices moe_group_kernel makes
 constexpr int kMoeFusedExperts = 256, kMoeFusedTop = 16;  // the one-token form
 
 // One wave: f(k, expert) for the `top` largest of z[0 .. E), largest first, the lower index first among equals (uniform)
@@ -51,28 +52,45 @@ __device__ __forceinline__ void wave_route(const float* z, int E, int top, int& 
     weight = p / wave_sum(p);
 }
 
+// one wave: the choice of row m
+struct MoeRoute {
+    const float* z;  // [M][E]
+    const RowRef* rows;
+    int M, E, top;
+    int32_t* sel;  // [M][top], -1 for padding rows: no pairs
+    float* wsel;
+};
 template <int NV>
-__global__ void __launch_bounds__(256) moe_topk_kernel(const float* __restrict__ z, const RowRef* __restrict__ rows, int M,
-                                                       int E, int top, int32_t* __restrict__ sel, float* __restrict__ wsel) {
-    const int m = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    if (m >= M) return;
+__device__ __forceinline__ void moe_route_row(const MoeRoute& r, int m) {
+    const int lane = threadIdx.x & 63;
     int e;
     float w;
-    wave_route<NV>(z + (size_t)m * E, E, top, e, w);
-    if (lane < top) {
-        sel[(size_t)m * top + lane] = rows[m].slot < 0 ? -1 : e;  // padding rows: no pairs
-        wsel[(size_t)m * top + lane] = w;
+    wave_route<NV>(r.z + (size_t)m * r.E, r.E, r.top, e, w);
+    if (lane < r.top) {
+        r.sel[(size_t)m * r.top + lane] = r.rows[m].slot < 0 ? -1 : e;
+        r.wsel[(size_t)m * r.top + lane] = w;
     }
+}
+template <int NV>
+__global__ void __launch_bounds__(256) moe_topk_kernel(MoeRoute r) {
+    const int m = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (m < r.M) moe_route_row<NV>(r, m);
 }
 
 // Pairs p = token * top + k with sel[p] = expert, in expert order: at[p] = row of the pair, rowmap[row] = token, each
 // expert's rows from a multiple of bm on (rows that fill up its last block read token 0), tiles[i] = {expert, first row}.
-// One workgroup; wave w handles experts w, w + 16, ...
-static __global__ void __launch_bounds__(1024) moe_group_kernel(const int32_t* __restrict__ sel, int P, int top, int E, int bm,
-                                                         int32_t* __restrict__ at, int32_t* __restrict__ rowmap,
-                                                         int2* __restrict__ tiles, int32_t* __restrict__ ntiles) {
+// One workgroup; wave w handles experts w, w + 16, ... NV > 0 (few rows): it also makes the choices, a wave per row.
+template <int NV>
+__global__ void __launch_bounds__(1024) moe_group_kernel(MoeRoute r, int bm, int32_t* __restrict__ at,
+                                                         int32_t* __restrict__ rowmap, int2* __restrict__ tiles,
+                                                         int32_t* __restrict__ ntiles) {
     __shared__ int base[kMoeMaxExperts + 1];  // first block of each expert
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, P = r.M * r.top, top = r.top, E = r.E;
+    const int32_t* sel = r.sel;
+    if constexpr (NV > 0) {
+        for (int m = wave; m < r.M; m += 16) moe_route_row<NV>(r, m);
+        __syncthreads();
+    }
     for (int e = wave; e < E; e += 16) {
         int n = 0;
         for (int p0 = 0; p0 < P; p0 += 64) n += (int)__popcll(__ballot(p0 + lane < P && sel[p0 + lane] == e));
@@ -99,7 +117,7 @@ static __global__ void __launch_bounds__(1024) moe_group_kernel(const int32_t* _
             }
             n += (int)__popcll(b);
         }
-        for (int r = r0 + n + lane; r < r1; r += 64) rowmap[r] = 0;
+        for (int i = r0 + n + lane; i < r1; i += 64) rowmap[i] = 0;
         for (int t = base[e] + lane; t < base[e + 1]; t += 64) tiles[t] = make_int2(e, t * bm);
     }
 }
