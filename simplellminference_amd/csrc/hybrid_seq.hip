@@ -567,7 +567,14 @@ struct SeqRec : HyProj<WT> {
         if (d.experts == 0) return SLI_OK;
 
         const void* xin = half ? (const void*)q().xh : (const void*)s->x;
-        HY_TRY(project(l.wg2, xin, s->Dp, l.n2, 0, gate_epi(l)));
+        if constexpr (half) {
+            HY_TRY(project(l.wg2, xin, s->Dp, np, 0, gate_epi(l)));
+            hipLaunchKernelGGL(moe_router_kernel, dim3(M / 16, (d.experts + 15) / 16), dim3(256), 0, st(),
+                               (const __half*)l.wg2 + (size_t)l.z0 * s->Dp, q().xh, l.zb, s->Dp, (int)d.experts, q().z);
+            SLI_HIP(hipGetLastError());
+        } else {
+            HY_TRY(project(l.wg2, xin, s->Dp, l.n2, 0, gate_epi(l)));
+        }
         const int E = d.experts, top = d.top, bm = bm_for(s, M, top, E), mt = moe_max_tiles(M * top, E, bm);
         const MoeRoute mr{q().z, s->rows, M, E, top, q().sel, q().wsel};
         HY_TRY(E <= 64 ? route<1>(mr, bm) : E <= 256 ? route<4>(mr, bm) : route<kMoeMaxExperts / 64>(mr, bm));

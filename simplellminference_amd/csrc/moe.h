@@ -7,6 +7,7 @@
 //     rows as one matrix, and moe_down_kernel sums the experts' down projections as column parts of one GEMV.
 // Weights: gate / up [E][ffp pairs {gate i, up i}][Dp], down [E][Dn][FFp].
 #pragma once
+#include "attn_mfma.h"
 #include "canon.h"
 #include "common.h"
 #include "gemv.h"
@@ -91,9 +92,23 @@ __global__ void __launch_bounds__(1024) moe_group_kernel(MoeRoute r, int bm, int
         for (int m = wave; m < r.M; m += 16) moe_route_row<NV>(r, m);
         __syncthreads();
     }
+    constexpr int kU = 8;  // loads in flight
+    int se[kU];
+    auto load = [&](int p0) {  // pairs p0 + 64 j + lane (-1 past the last)
+#pragma unroll
+        for (int j = 0; j < kU; ++j) {
+            const int p = p0 + 64 * j + lane;
+            se[j] = sel[min(p, P - 1)];
+            if (p >= P) se[j] = -1;
+        }
+    };
     for (int e = wave; e < E; e += 16) {
         int n = 0;
-        for (int p0 = 0; p0 < P; p0 += 64) n += (int)__popcll(__ballot(p0 + lane < P && sel[p0 + lane] == e));
+        for (int p0 = 0; p0 < P; p0 += 64 * kU) {
+            load(p0);
+#pragma unroll
+            for (int j = 0; j < kU; ++j) n += (int)__popcll(__ballot(se[j] == e));
+        }
         if (lane == 0) base[e + 1] = (n + bm - 1) / bm;
     }
     __syncthreads();
@@ -106,21 +121,62 @@ __global__ void __launch_bounds__(1024) moe_group_kernel(MoeRoute r, int bm, int
     for (int e = wave; e < E; e += 16) {
         const int r0 = base[e] * bm, r1 = base[e + 1] * bm;
         int n = 0;
-        for (int p0 = 0; p0 < P && r1 > r0; p0 += 64) {
-            const int p = p0 + lane;
-            const bool mine = p < P && sel[p] == e;
-            const unsigned long long b = __ballot(mine);
-            if (mine) {
-                const int row = r0 + n + (int)__popcll(b & ((1ull << lane) - 1));
-                at[p] = row;
-                rowmap[row] = p / top;
+        for (int p0 = 0; p0 < P && r1 > r0; p0 += 64 * kU) {
+            load(p0);
+#pragma unroll
+            for (int j = 0; j < kU; ++j) {
+                const bool mine = se[j] == e;
+                const unsigned long long b = __ballot(mine);
+                if (mine) {
+                    const int p = p0 + 64 * j + lane, row = r0 + n + (int)__popcll(b & ((1ull << lane) - 1));
+                    at[p] = row;
+                    rowmap[row] = p / top;
+                }
+                n += (int)__popcll(b);
             }
-            n += (int)__popcll(b);
         }
         for (int i = r0 + n + lane; i < r1; i += 64) rowmap[i] = 0;
         for (int t = base[e] + lane; t < base[e + 1]; t += 64) tiles[t] = make_int2(e, t * bm);
     }
 }
+// Router logits of a prompt's rows, z[m][e] = w[e] . x[m] + b[e] (few rows of weights: as part of a wide GEMM they would
+// cost a column of its tiles). Grid (M / 16, E / 16), 4 waves that split K: A = 16 experts' rows, B = 16 tokens, both
+// straight from memory.
+static __global__ void __launch_bounds__(256) moe_router_kernel(const __half* __restrict__ w, const __half* __restrict__ x,
+                                                                const float* __restrict__ b, int K, int E, float* __restrict__ z) {
+    constexpr int kU = 8;
+    __shared__ float4 red[3][64];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, i16 = lane & 15, g = lane >> 4;
+    const int e0 = blockIdx.y * 16, m = blockIdx.x * 16 + i16;
+    const int nkb = K / 32, kb0 = nkb * wave / 4, kb1 = nkb * (wave + 1) / 4;
+    const __half* wp = w + (size_t)min(e0 + i16, E - 1) * K + 8 * g;
+    const __half* xp = x + (size_t)m * K + 8 * g;
+    am_float4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
+    for (int k0 = kb0; k0 < kb1; k0 += kU) {
+        u32x4 a[kU], v[kU];
+#pragma unroll
+        for (int j = 0; j < kU; ++j) {
+            const int kb = min(k0 + j, kb1 - 1);
+            a[j] = load16<false>(wp + 32 * kb);
+            v[j] = load16<false>(xp + 32 * kb);
+        }
+#pragma unroll
+        for (int j = 0; j < kU; ++j)
+            if (k0 + j < kb1) acc = am_mfma(a[j], v[j], acc);
+    }
+    if (wave > 0) red[wave - 1][lane] = make_float4(acc[0], acc[1], acc[2], acc[3]);
+    __syncthreads();
+    if (wave > 0) return;
+#pragma unroll
+    for (int i = 0; i < 3; ++i) {
+        const float4 r = red[i][lane];
+        acc[0] += r.x, acc[1] += r.y, acc[2] += r.z, acc[3] += r.w;
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+        if (e0 + 4 * g + i < E) z[(size_t)m * E + e0 + 4 * g + i] = acc[i] + b[e0 + 4 * g + i];
+}
+
 // row blocks P pairs can need
 inline int moe_max_tiles(int P, int E, int bm) { return P / bm + std::min(E, P); }
 
