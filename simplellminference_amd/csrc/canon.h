@@ -99,8 +99,8 @@ __global__ void __launch_bounds__(256) canon_rows_kernel(CanonArgs a, OT* c1, OT
 }
 
 // The same for kCanonFusedTaps taps and ld <= 4 * blockDim.x: one float4 of a row per thread, every row and coefficient
-// in flight at once, the rows' sums in one exchange.
-template <typename OT>
+// in flight at once, the rows' sums in one exchange. RAW: CanonArgs::raw.
+template <typename OT, bool RAW>
 __global__ void __launch_bounds__(1024) canon4_rows_kernel(CanonArgs a, OT* c1, OT* c2, int write_ring) {
     constexpr int TAPS = kCanonFusedTaps;
     __shared__ float red[16][TAPS];
@@ -122,38 +122,47 @@ __global__ void __launch_bounds__(1024) canon4_rows_kernel(CanonArgs a, OT* c1, 
                                     : j <= nall ? ring + (size_t)((r.pos - j) % TAPS) * a.ld : a.x + (size_t)m * a.ld;
         n[j] = reinterpret_cast<const float4*>(src)[i];
         f1[j] = reinterpret_cast<const float4*>(a.f1 + (size_t)j * a.ld)[i];
-        f2[j] = reinterpret_cast<const float4*>((a.f2 ? a.f2 : a.f1) + (size_t)j * a.ld)[i];
+        if constexpr (!RAW) f2[j] = reinterpret_cast<const float4*>((c2 ? a.f2 : a.f1) + (size_t)j * a.ld)[i];
     }
-    if (!a.raw) {
+    float4 s1 = make_float4(0.f, 0.f, 0.f, 0.f), s2 = s1;
+    if constexpr (RAW) {
+#pragma unroll
+        for (int j = TAPS - 1; j >= 0; --j)  // (selects, no branches: the loads stay together)
+            s1 = fma4(n[j], mul4(f1[j], j <= nall ? 1.0f : 0.0f), s1);
+        s2 = n[0];
+    } else {
 #pragma unroll
         for (int j = 0; j < TAPS; ++j) {
             const float ss = wave_sum(tid < n4 ? sq4(n[j]) : 0.0f);
             if ((tid & 63) == 0) red[tid >> 6][j] = ss;
         }
         __syncthreads();
-    }
-    float4 s1 = make_float4(0.f, 0.f, 0.f, 0.f), s2 = s1;
 #pragma unroll
-    for (int j = TAPS - 1; j >= 0; --j) {
-        if (j > nall) continue;
-        if (j <= nin && !a.raw) {
-            float t = 0.0f;
-            for (int w = 0; w < (int)blockDim.x / 64; ++w) t += red[w][j];
-            n[j] = mul4(n[j], 1.0f / sqrtf(t / (float)a.D + a.eps));
+        for (int j = TAPS - 1; j >= 0; --j) {
+            if (j > nall) continue;
+            if (j <= nin) {
+                float t = 0.0f;
+                for (int w = 0; w < (int)blockDim.x / 64; ++w) t += red[w][j];
+                n[j] = mul4(n[j], 1.0f / sqrtf(t / (float)a.D + a.eps));
+            }
+            s1 = fma4(n[j], f1[j], s1);
+            s2 = fma4(n[j], f2[j], s2);
         }
-        s1 = fma4(n[j], f1[j], s1);
-        s2 = fma4(n[j], f2[j], s2);
     }
     if (tid >= n4) return;
     if (write_ring) reinterpret_cast<float4*>(ring + (size_t)(r.pos % TAPS) * a.ld)[i] = n[0];
     store4(c1 + (size_t)m * a.ld + 4 * i, s1);
-    if (c2) store4(c2 + (size_t)m * a.ld + 4 * i, a.f2 ? s2 : n[0]);
+    if (c2) store4(c2 + (size_t)m * a.ld + 4 * i, s2);
 }
 
 template <typename OT>
 hipError_t launch_canon_rows(const CanonArgs& a, OT* c1, OT* c2, int write_ring, hipStream_t s) {
-    if (a.taps == kCanonFusedTaps && a.ld <= 4096)
-        hipLaunchKernelGGL(canon4_rows_kernel<OT>, dim3(a.M), dim3((a.ld / 4 + 63) / 64 * 64), 0, s, a, c1, c2, write_ring);
+    const dim3 bl((a.ld / 4 + 63) / 64 * 64);
+    const bool four = a.taps == kCanonFusedTaps && a.ld <= 4096;
+    if (four && a.raw)
+        hipLaunchKernelGGL((canon4_rows_kernel<OT, true>), dim3(a.M), bl, 0, s, a, c1, c2, write_ring);
+    else if (four)
+        hipLaunchKernelGGL((canon4_rows_kernel<OT, false>), dim3(a.M), bl, 0, s, a, c1, c2, write_ring);
     else
         hipLaunchKernelGGL(canon_rows_kernel<OT>, dim3(a.M), dim3(256), 0, s, a, c1, c2, write_ring);
     return hipGetLastError();
