@@ -68,6 +68,7 @@ MODELS = {
     "ranks-to-256": stack(blk(kv_rank=130, window=90), blk(kv_rank=192), blk(kv_rank=256, heads=33, dim=4, vdim=4)),
     "ranks-to-448": stack(blk(kv_rank=320), blk(kv_rank=400, window=66), blk(kv_rank=448, window=100)),
     "ranks-past-512": stack(blk(kv_rank=512, window=70), blk(kv_rank=530, window=80)),
+    "ranks-past-1024": stack(blk(kv_rank=1100, window=70)),
     "whole-context": stack(blk(window=0), blk(window=500)),
     "long-taps": stack(blk(), blk(experts=0), taps=7),
     "four-taps": stack(blk(), blk(), taps=4, order=[0, 1, 0]),
@@ -153,12 +154,14 @@ def test_window_edges(gpu, window, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("place", [0, 63, 64, 255, 256, 700, 1023, 1024])
-def test_far_key_in_a_long_window(gpu, place, dtype):
+@pytest.mark.parametrize("place,heads,rank", [(p, 18, 96) for p in (0, 63, 64, 255, 256, 700, 1023, 1024)] +
+                         [(p, 3, 500) for p in (0, 64, 1100)])
+def test_far_key_in_a_long_window(gpu, place, heads, rank, dtype):
     """One key among many hundred, at tile, split and pass borders, found from a prompt row in a later pass and from
-    decoded rows; more heads than one workgroup of the decode attention takes."""
+    decoded rows; more heads than one workgroup of the decode attention takes, or a rank so large that the merge of its
+    splits takes more than one round of loads."""
     n = 1300
-    c, t = strong_pair(n, n, 18, 96)
+    c, t = strong_pair(n, n, heads, rank)
     t["l0.mix.uk"] = t["l0.mix.uk"] * 2
     ids = [0] * n
     ids[place] = 2
